@@ -72,6 +72,10 @@ enum {
     MOON_EPI_BIAS_GELU = 2  /* C = gelu(f16(f16(acc)+bias))  + ops.gelu, ops.zig:1635-1774 */
 };
 
+/* element type of a decoder opened from a model folder: storage of weights, cache and activations between kernels.  The
+ * residual stream, norms, scores, routers and accumulators are f32 either way; F32 computes everything in f32. */
+enum { MOON_DTYPE_BF16 = 0, MOON_DTYPE_F32 = 1 };
+
 /* layout of the B operand */
 enum {
     MOON_B_KN = 0, /* B[K,N] row-major: hgemm.matmul (vision weights, weights.zig:459-474) */
@@ -268,6 +272,26 @@ int moon_text_model_create(moon_ctx *ctx, const moon_text_config *cfg, const moo
  * (seed, stream = declaration order above), LayerNorm gamma = 1, beta = 0. */
 int moon_text_model_create_synthetic(moon_ctx *ctx, const moon_text_config *cfg, uint64_t seed, float std_dev,
                                      moon_text_model **out);
+/* A decoder from a model folder: dir/config.json names the design ("architecture", looked up in the library's registry) and
+ * describes its layers, dir/model.safetensors holds the weights.  The session is a moon_text_model like any other (forward,
+ * greedy, sample, generate, next_token, reset, position); what only the fixed f16 block has (forward_embeds, embed, f16 logits
+ * and hidden rows, decode modes, the per-kernel profile) is refused with MOON_EINVAL.  max_seq: the longest sequence; it sizes
+ * the cache of layers that see everything, a windowed layer keeps its window and one call's rows.  No counterpart in the
+ * reference, which has one decoder.  A folder the registry or the reader refuses is MOON_EFORMAT / MOON_ESHAPE. */
+int moon_text_model_open(moon_ctx *ctx, const char *dir, int dtype, size_t max_seq, moon_text_model **out);
+/* The same with random weights generated on the device (matrices ~N(0,std)) for the text of a config.json; every size must
+ * be a multiple of 64, head sizes of 8. */
+int moon_text_model_open_synthetic(moon_ctx *ctx, const char *config_json, int dtype, size_t max_seq, uint64_t seed, float std_dev,
+                                   moon_text_model **out);
+/* Names of the registered designs, separated by ", ". */
+const char *moon_text_designs(void);
+size_t moon_text_vocab(const moon_text_model *m);
+size_t moon_text_dim(const moon_text_model *m);
+/* moon_text_forward that also brings back logits: logits[i] (f32 [vocab]) belong to token want[i] of this call. */
+int moon_text_forward_logits(moon_text_model *m, const uint32_t *ids, size_t n_ids, const size_t *want, size_t n_want, float *logits);
+/* moon_text_logits / moon_text_hidden in f32 (the residual stream is f32 where the design keeps it so). */
+int moon_text_logits_f32(moon_text_model *m, float *logits);
+int moon_text_hidden_f32(moon_text_model *m, float *hidden, size_t n_rows);
 void moon_text_model_destroy(moon_text_model *m);
 /* KVCache.reset (text_model.zig:526-530). */
 int moon_text_reset(moon_text_model *m);

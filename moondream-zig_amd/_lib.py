@@ -17,6 +17,7 @@ HEADER_PATH = os.path.join(os.path.dirname(_HERE), "include", "moonhip.h")
 # error codes (moonhip.h)
 OK, EINVAL_DIM, ESHAPE, ESEQ_TOO_LONG, ENOMEM, EHIP, EINVAL, EROT_DIM, ETOKEN, EEPS, ENODEVICE, EFORMAT, ETEMPERATURE = range(13)
 SAMPLE_GREEDY, SAMPLE_MULTINOMIAL, SAMPLE_TOP_K, SAMPLE_MIN_P = range(4)
+DTYPE_BF16, DTYPE_F32 = 0, 1
 EPI_NONE, EPI_BIAS, EPI_BIAS_GELU = 0, 1, 2
 B_KN, B_NK = 0, 1
 
@@ -114,6 +115,14 @@ SIGNATURES = {
     "moon_text_config_default": (None, [C.POINTER(TextConfig)]),
     "moon_text_model_create": (_i, [_vp, C.POINTER(TextConfig), C.POINTER(TextWeights), _pp]),
     "moon_text_model_create_synthetic": (_i, [_vp, C.POINTER(TextConfig), _u64, _f, _pp]),
+    "moon_text_model_open": (_i, [_vp, C.c_char_p, _i, _sz, _pp]),
+    "moon_text_model_open_synthetic": (_i, [_vp, C.c_char_p, _i, _sz, _u64, _f, _pp]),
+    "moon_text_designs": (C.c_char_p, []),
+    "moon_text_vocab": (_sz, [_vp]),
+    "moon_text_dim": (_sz, [_vp]),
+    "moon_text_forward_logits": (_i, [_vp, _vp, _sz, _vp, _sz, _vp]),
+    "moon_text_logits_f32": (_i, [_vp, _vp]),
+    "moon_text_hidden_f32": (_i, [_vp, _vp, _sz]),
     "moon_text_model_destroy": (None, [_vp]),
     "moon_text_reset": (_i, [_vp]),
     "moon_text_forward": (_i, [_vp, _vp, _sz]),

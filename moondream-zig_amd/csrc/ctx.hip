@@ -242,7 +242,7 @@ static inline uint64_t stream_key(uint64_t seed, uint64_t stream) {
     return mix64(mix64(seed + 0x9E3779B97F4A7C15ull) ^ (stream * 0xD1B54A32D192ED03ull + 0x2545F4914F6CDD1Dull));
 }
 
-__global__ void fill_normal_kernel(half_t *dst, size_t n, uint64_t key, float scale) {
+template <class T> __global__ void fill_normal_kernel(T *dst, size_t n, uint64_t key, float scale) {
     size_t i = size_t(blockIdx.x) * blockDim.x + threadIdx.x;
     const size_t stride = size_t(gridDim.x) * blockDim.x;
     for (; i < n; i += stride) {
@@ -256,7 +256,7 @@ __global__ void fill_normal_kernel(half_t *dst, size_t n, uint64_t key, float sc
         const int32_t c = int32_t(s) - 262140;
         float f = float(c) * scale; // rounded to f32 first, then to f16, like the host generator
         asm volatile("" : "+v"(f));  // keeps the multiply from being folded into a single-rounding f16 convert
-        dst[i] = (half_t)f;
+        dst[i] = (T)f;
     }
 }
 
@@ -280,7 +280,16 @@ static inline unsigned fill_grid(size_t n) {
 int launch_fill_normal(moon_ctx *ctx, half_t *dst, size_t n, uint64_t seed, uint64_t stream, float std_dev) {
     if (!n) return MOON_OK;
     const float scale = std_dev * (1.0f / 53510.105f);
-    hipLaunchKernelGGL(fill_normal_kernel, dim3(fill_grid(n)), dim3(256), 0, ctx->stream, dst, n, stream_key(seed, stream), scale);
+    hipLaunchKernelGGL(fill_normal_kernel<half_t>, dim3(fill_grid(n)), dim3(256), 0, ctx->stream, dst, n, stream_key(seed, stream), scale);
+    MOON_HIP(ctx, hipGetLastError());
+    return MOON_OK;
+}
+int launch_fill_normal_t(moon_ctx *ctx, int dtype, void *dst, size_t n, uint64_t seed, uint64_t stream, float std_dev) {
+    if (!n) return MOON_OK;
+    const float scale = std_dev * (1.0f / 53510.105f);
+    if (dtype == MOON_DTYPE_BF16)
+        hipLaunchKernelGGL(fill_normal_kernel<bf16_t>, dim3(fill_grid(n)), dim3(256), 0, ctx->stream, (bf16_t *)dst, n, stream_key(seed, stream), scale);
+    else hipLaunchKernelGGL(fill_normal_kernel<float>, dim3(fill_grid(n)), dim3(256), 0, ctx->stream, (float *)dst, n, stream_key(seed, stream), scale);
     MOON_HIP(ctx, hipGetLastError());
     return MOON_OK;
 }

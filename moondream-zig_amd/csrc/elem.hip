@@ -43,7 +43,7 @@ __global__ void residual2_kernel(half_t *hidden, const half_t *__restrict__ attn
 // sampling.argmax (sampling.zig:257-273): strict '>' scan from index 0, i.e. the lowest index among
 // equal maxima; NaN never wins.  Single workgroup (51200 logits = 100 KiB).
 template <class T>
-__global__ __launch_bounds__(1024) void argmax_kernel(const T *__restrict__ logits, int n, uint32_t *out) {
+__global__ __launch_bounds__(1024) void argmax_kernel(const T *__restrict__ logits, int n, uint32_t *out, uint32_t *state, uint32_t *out_ids) {
     __shared__ float sv[16];
     __shared__ int si[16];
     float best = -INFINITY;
@@ -83,7 +83,9 @@ __global__ __launch_bounds__(1024) void argmax_kernel(const T *__restrict__ logi
         // the reference starts from max_val = data[0], max_idx = 0: if nothing compares greater
         // (all NaN, or all -inf) index 0 is returned
         const float first = (float)logits[0];
-        *out = (idx == 0x7fffffff || first != first) ? 0u : (uint32_t)idx; // a NaN at index 0 is never displaced
+        const uint32_t tok = (idx == 0x7fffffff || first != first) ? 0u : (uint32_t)idx; // a NaN at index 0 is never displaced
+        if (out) *out = tok;
+        if (state) record_token(state, out_ids, tok, 0u);
     }
 }
 
@@ -303,13 +305,19 @@ int launch_image_patches(moon_ctx *ctx, const uint8_t *image, half_t *out, size_
 
 int launch_argmax(moon_ctx *ctx, const half_t *logits, size_t n, uint32_t *index_out) {
     if (!n || n > 0x7fffffff) return moon_fail(ctx, MOON_EINVAL, "argmax: empty or oversized tensor");
-    hipLaunchKernelGGL(argmax_kernel<half_t>, dim3(1), dim3(1024), 0, ctx->stream, logits, (int)n, index_out);
+    hipLaunchKernelGGL(argmax_kernel<half_t>, dim3(1), dim3(1024), 0, ctx->stream, logits, (int)n, index_out, nullptr, nullptr);
     MOON_HIP(ctx, hipGetLastError());
     return MOON_OK;
 }
 int launch_argmax_f32(moon_ctx *ctx, const float *logits, size_t n, uint32_t *index_out) {
     if (!n || n > 0x7fffffff) return moon_fail(ctx, MOON_EINVAL, "argmax: empty or oversized tensor");
-    hipLaunchKernelGGL(argmax_kernel<float>, dim3(1), dim3(1024), 0, ctx->stream, logits, (int)n, index_out);
+    hipLaunchKernelGGL(argmax_kernel<float>, dim3(1), dim3(1024), 0, ctx->stream, logits, (int)n, index_out, nullptr, nullptr);
+    MOON_HIP(ctx, hipGetLastError());
+    return MOON_OK;
+}
+int launch_argmax_record_f32(moon_ctx *ctx, const float *logits, size_t n, uint32_t *state, uint32_t *out_ids) {
+    if (!n || n > 0x7fffffff) return moon_fail(ctx, MOON_EINVAL, "argmax: empty or oversized tensor");
+    hipLaunchKernelGGL(argmax_kernel<float>, dim3(1), dim3(1024), 0, ctx->stream, logits, (int)n, nullptr, state, out_ids);
     MOON_HIP(ctx, hipGetLastError());
     return MOON_OK;
 }

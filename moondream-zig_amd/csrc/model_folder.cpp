@@ -1,0 +1,200 @@
+// Model folders (config.json + model.safetensors) and the registry of designs that are described as a list of layers.
+#include "model_folder.hpp"
+
+#include <fcntl.h>
+#include <sys/mman.h>
+#include <sys/stat.h>
+#include <unistd.h>
+
+#include <cerrno>
+
+// ------------------------------------------------------------------ safetensors
+SafeTensors::~SafeTensors() {
+    if (map) munmap(map, size);
+}
+
+int SafeTensors::open(const std::string &path, std::string *err) {
+    const int fd = ::open(path.c_str(), O_RDONLY);
+    struct stat st;
+    if (fd < 0 || fstat(fd, &st) != 0) {
+        *err = path + ": " + strerror(errno);
+        if (fd >= 0) close(fd);
+        return MOON_EINVAL;
+    }
+    size = (size_t)st.st_size;
+    map = size >= 8 ? mmap(nullptr, size, PROT_READ, MAP_PRIVATE, fd, 0) : MAP_FAILED;
+    close(fd);
+    if (map == MAP_FAILED) {
+        map = nullptr;
+        *err = path + ": not a safetensors file";
+        return MOON_EFORMAT;
+    }
+    const unsigned char *p = (const unsigned char *)map;
+    uint64_t header = 0;
+    for (int i = 7; i >= 0; i--) header = header << 8 | p[i];
+    Json j;
+    if (header > size - 8 || !Json::parse((const char *)p + 8, (size_t)header, &j, err) || j.type != Json::OBJECT) {
+        *err = path + ": bad header " + *err;
+        return MOON_EFORMAT;
+    }
+    const size_t base = 8 + (size_t)header;
+    for (const auto &m : j.members) {
+        if (m.first == "__metadata__") continue;
+        const Json *dt = m.second.find("dtype"), *sh = m.second.find("shape"), *off = m.second.find("data_offsets");
+        StTensor t;
+        bool ok = dt && dt->type == Json::STRING && sh && sh->type == Json::ARRAY && off && off->type == Json::ARRAY && off->items.size() == 2 &&
+                  off->items[0].is_size() && off->items[1].is_size();
+        if (ok) {
+            t.dtype = dt->str;
+            const size_t el = t.dtype == "BF16" || t.dtype == "F16" ? 2 : t.dtype == "F32" || t.dtype == "I32" ? 4 : 0;
+            unsigned __int128 n = 1;
+            for (const Json &d : sh->items) {
+                ok = ok && d.is_size();
+                t.shape.push_back(ok ? (size_t)d.num : 0);
+                n *= t.shape.back();
+                ok = ok && n < ((unsigned __int128)1 << 62);
+            }
+            const size_t a = (size_t)off->items[0].num, b = (size_t)off->items[1].num;
+            ok = ok && el && a <= b && b <= size - base && n * el == b - a;
+            t.data = p + base + a;
+            t.bytes = b - a;
+        }
+        if (!ok) {
+            *err = path + ": tensor '" + m.first + "' does not fit its header entry";
+            return MOON_EFORMAT;
+        }
+        tensors[m.first] = t;
+    }
+    return MOON_OK;
+}
+
+const StTensor *SafeTensors::find(const std::string &name) const {
+    const auto it = tensors.find(name);
+    return it == tensors.end() ? nullptr : &it->second;
+}
+
+// ------------------------------------------------------------------ config.json
+namespace {
+
+struct Fields { // typed access to a config's members; the first failure is kept
+    std::string *err;
+    bool ok = true;
+    bool fail(const std::string &what) {
+        if (ok) *err = "config.json: " + what;
+        return ok = false;
+    }
+    const Json *object(const Json &j, const char *key, const std::string &where) {
+        const Json *v = j.find(key);
+        if (!v || v->type != Json::OBJECT) fail(where + key + " is missing or no object");
+        return v && v->type == Json::OBJECT ? v : nullptr;
+    }
+    size_t size(const Json *j, const char *key, const std::string &where) {
+        const Json *v = j ? j->find(key) : nullptr;
+        if (!v || !v->is_size() || v->num < 1 || v->num > 1e9) {
+            fail(where + key + " is missing or no positive integer");
+            return 1;
+        }
+        return (size_t)v->num;
+    }
+    float number(const Json *j, const char *key, const std::string &where) {
+        const Json *v = j ? j->find(key) : nullptr;
+        if (!v || v->type != Json::NUMBER) {
+            fail(where + key + " is missing or no number");
+            return 1.0f;
+        }
+        return (float)v->num;
+    }
+};
+
+std::string indexed(const char *prefix, size_t i, const std::string &rest) { return prefix + std::to_string(i) + rest; }
+
+// Rikanex: parallel layers of windowed attention without positions (unit-RMS q and k, sink, output gate, values mixed with the
+// first layer's) and a gated feed-forward, dense or of routed experts.
+bool parse_rikanex(const Json &c, LayerListSpec *s, std::string *err) {
+    Fields f{err};
+    s->vocab = f.size(&c, "vocab", "");
+    s->width = f.size(&c, "width", "");
+    s->embed_scale = f.number(f.object(c, "embedding", ""), "scale", "embedding.");
+    s->eps = f.number(f.object(c, "norm", ""), "eps", "norm.");
+    if (!(s->eps > 0.0f)) f.fail("norm.eps must be positive");
+    const Json *layers = c.find("layers");
+    if (!layers || layers->type != Json::ARRAY || layers->items.empty()) return f.fail("layers is missing or empty");
+    for (size_t i = 0; i < layers->items.size() && f.ok; i++) {
+        const Json &l = layers->items[i];
+        const std::string at = "layers[" + std::to_string(i) + "].";
+        LayerSpec spec;
+        const Json *type = l.find("type");
+        if (!type || type->str != "attention") return f.fail(at + "type is not 'attention'");
+        const Json *m = f.object(l, "mixer", at);
+        MixerSpec &mx = spec.mixer;
+        mx.heads = f.size(m, "heads", at + "mixer.");
+        mx.kv_heads = f.size(m, "kv_heads", at + "mixer.");
+        mx.dim = f.size(m, "dim", at + "mixer.");
+        mx.vdim = f.size(m, "vdim", at + "mixer.");
+        mx.scale = f.number(m, "scale", at + "mixer.");
+        if (mx.heads % mx.kv_heads) f.fail(at + "mixer.kv_heads does not divide heads");
+        const Json *mask = m ? m->find("mask") : nullptr, *mix = m ? m->find("v_mix") : nullptr;
+        if (mask && mask->type != Json::NIL) mx.window = f.size(mask, "size", at + "mixer.mask.");
+        mx.v_mix = mix && mix->type == Json::BOOL && mix->b;
+        mx.qk_rms = mx.sink = mx.gate = true;
+        const Json *mlp = l.find("mlp");
+        if (mlp && mlp->type != Json::NIL) {
+            const Json *kind = mlp->find("kind");
+            if (kind && kind->str == "dense") {
+                spec.ff.kind = FeedForwardSpec::DENSE;
+                spec.ff.ff = f.size(mlp, "ff", at + "mlp.");
+            } else if (kind && kind->str == "moe") {
+                spec.ff.kind = FeedForwardSpec::EXPERTS;
+                spec.ff.ff = f.size(f.object(*mlp, "expert", at + "mlp."), "ff", at + "mlp.expert.");
+                const Json *router = f.object(*mlp, "router", at + "mlp.");
+                spec.ff.experts = f.size(router, "experts", at + "mlp.router.");
+                spec.ff.top = f.size(router, "top", at + "mlp.router.");
+                if (spec.ff.top > spec.ff.experts) f.fail(at + "mlp.router.top exceeds experts");
+            } else f.fail(at + "mlp.kind is neither 'dense' nor 'moe'");
+        }
+        s->layers.push_back(spec);
+    }
+    return f.ok;
+}
+
+const TensorNames RIKANEX_NAMES = {
+    [] { return std::string("embed"); },
+    [] { return std::string("head"); },
+    [] { return std::string("final.norm"); },
+    [](size_t i) { return indexed("l", i, ".norm1"); },
+    [](size_t i, const char *what) { return indexed("l", i, std::string(".mix.") + what); },
+    [](size_t i, const char *what) { return indexed("l", i, std::string(".mlp.") + what); },
+    [](size_t i, size_t e, const char *what) { return indexed("l", i, indexed(".mlp.e", e, std::string(".") + what)); },
+    ".b",
+};
+
+const Design DESIGNS[] = {
+    {"Rikanex", parse_rikanex, RIKANEX_NAMES},
+};
+
+} // namespace
+
+const Design *find_design(const std::string &architecture) {
+    for (const Design &d : DESIGNS)
+        if (architecture == d.name) return &d;
+    return nullptr;
+}
+
+std::string known_designs() {
+    std::string s;
+    for (const Design &d : DESIGNS) s += std::string(s.empty() ? "" : ", ") + d.name;
+    return s;
+}
+
+int parse_model_config(const char *text, size_t len, const Design **design, LayerListSpec *spec, std::string *err) {
+    Json c;
+    if (!Json::parse(text, len, &c, err)) return MOON_EFORMAT;
+    const Json *a = c.find("architecture");
+    *design = a && a->type == Json::STRING ? find_design(a->str) : nullptr;
+    if (!*design) {
+        *err = "config.json: architecture '" + (a ? a->str : std::string()) + "' is not one of: " + known_designs();
+        return MOON_EFORMAT;
+    }
+    spec->design = (*design)->name;
+    return (*design)->parse(c, spec, err) ? MOON_OK : MOON_EFORMAT;
+}

@@ -16,6 +16,8 @@ typedef _Float16 half_t;
 typedef _Float16 half2_t __attribute__((ext_vector_type(2)));
 typedef _Float16 half4_t __attribute__((ext_vector_type(4)));
 typedef _Float16 half8_t __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16_t;
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float float4_t __attribute__((ext_vector_type(4)));
 typedef float float16_t __attribute__((ext_vector_type(16)));
 
@@ -152,6 +154,8 @@ int launch_add(moon_ctx *ctx, half_t *a, const half_t *b, size_t n);
 // a = f16(a + f16(b + c))  -- the parallel-block residual (text_model.zig:170-171)
 int launch_residual2(moon_ctx *ctx, half_t *hidden, const half_t *attn, const half_t *mlp, size_t n);
 int launch_argmax(moon_ctx *ctx, const half_t *logits, size_t n, uint32_t *index_out);
+// argmax_f32 with the generation loop's bookkeeping (record_token, the position left where it is)
+int launch_argmax_record_f32(moon_ctx *ctx, const float *logits, size_t n, uint32_t *state, uint32_t *out_ids);
 int launch_argmax_f32(moon_ctx *ctx, const float *logits, size_t n, uint32_t *index_out);
 // resized u8 image [H,W,C] -> normalised f16 patches [copies * (H/P)*(W/P), C*P*P], rows `pitch` halfs apart
 int launch_image_patches(moon_ctx *ctx, const uint8_t *image, half_t *out, size_t H, size_t W, size_t C, size_t P, size_t copies, size_t pitch);
@@ -177,6 +181,8 @@ int launch_split_heads(moon_ctx *ctx, const half_t *qkv, size_t row_stride, size
                        size_t S, size_t H, size_t D);
 
 int launch_fill_normal(moon_ctx *ctx, half_t *dst, size_t n, uint64_t seed, uint64_t stream, float std_dev);
+// the same values as bf16 or f32 (dtype: a MOON_DTYPE_* value)
+int launch_fill_normal_t(moon_ctx *ctx, int dtype, void *dst, size_t n, uint64_t seed, uint64_t stream, float std_dev);
 int launch_fill_const(moon_ctx *ctx, half_t *dst, size_t n, float value);
 int launch_fill_uniform_u32(moon_ctx *ctx, uint32_t *dst, size_t n, uint64_t seed, uint64_t stream, uint32_t modulo);
 

@@ -4,7 +4,13 @@
 // weights.zig:439-454), which is already the k-contiguous [N,K] form both the GEMV and the GEMM kernels read.
 // Activations and the cache never leave the device; a decode step enqueues kernels only (token id and position
 // are read from device memory), so the loop needs no host synchronisation until the ids are fetched.
+//
+// Decoders that are described as a list of layers (layer_list.hpp) are sessions of the same kind: the position, the loop, the
+// sampler and the calls are these, the layers and the cache are the list's.
 #include "moon_internal.hpp"
+
+#include "layer_list.hpp"
+#include "model_folder.hpp"
 
 #include <cstdlib>
 #include <cstring>
@@ -92,6 +98,8 @@ struct moon_text_model {
     uint32_t lm_launches = 0;
     long long *layer_trace = nullptr; // [grid][8] stamps of the most recent layer launch when MOON_DECODE_TRACE is set
     struct StepProfiler *prof = nullptr;  // set only inside moon_text_greedy_profile
+    const float *logits_f32 = nullptr;    // the list's latest logits
+    LayerList *list = nullptr;            // set: the layers, cache, hidden rows and logits are the list's, everything of the fixed block is unused
     std::vector<void *> allocs;
 };
 
@@ -158,6 +166,19 @@ int check_cfg(moon_ctx *ctx, const moon_text_config *c) {
     return MOON_OK;
 }
 
+// what the calls and the generation loop need of any decoder: ids, random numbers, the loop's state, staging
+int alloc_loop(moon_text_model *m) {
+    const size_t S = m->cfg.max_seq;
+    MOON_TRY(dalloc_t(m, S, &m->ids_dev));
+    MOON_HIP(m->ctx, hipHostMalloc((void **)&m->ids_pinned, S * sizeof(uint32_t), hipHostMallocDefault));
+    MOON_HIP(m->ctx, hipHostMalloc((void **)&m->host_words, 64 * sizeof(uint32_t), hipHostMallocDefault));
+    MOON_HIP(m->ctx, hipHostMalloc((void **)&m->stage_up, STAGE_BYTES, hipHostMallocDefault));
+    MOON_HIP(m->ctx, hipHostMalloc((void **)&m->stage_down, STAGE_BYTES, hipHostMallocDefault));
+    MOON_TRY(dalloc_t(m, S, &m->u_dev));
+    MOON_TRY(dalloc_t(m, 8, &m->state_dev));
+    return launch_fill_uniform_u32(m->ctx, m->state_dev, 8, 0, 0, 1); // zeros
+}
+
 int alloc_all(moon_text_model *m) {
     const Sizes z = sizes(m->cfg);
     MOON_TRY(dalloc_t(m, z.V * z.d, &m->wte));
@@ -188,14 +209,7 @@ int alloc_all(moon_text_model *m) {
     MOON_TRY(dalloc_t(m, z.S * z.d, &m->mlp));
     MOON_TRY(dalloc_t(m, z.V, &m->logits));
     MOON_TRY(dalloc_t(m, z.d, &m->ln_last));
-    MOON_TRY(dalloc_t(m, z.S, &m->ids_dev));
-    MOON_HIP(m->ctx, hipHostMalloc((void **)&m->ids_pinned, z.S * sizeof(uint32_t), hipHostMallocDefault));
-    MOON_HIP(m->ctx, hipHostMalloc((void **)&m->host_words, 64 * sizeof(uint32_t), hipHostMallocDefault));
-    MOON_HIP(m->ctx, hipHostMalloc((void **)&m->stage_up, STAGE_BYTES, hipHostMallocDefault));
-    MOON_HIP(m->ctx, hipHostMalloc((void **)&m->stage_down, STAGE_BYTES, hipHostMallocDefault));
-    MOON_TRY(dalloc_t(m, z.S, &m->u_dev));
-    MOON_TRY(dalloc_t(m, 8, &m->state_dev));
-    MOON_TRY(launch_fill_uniform_u32(m->ctx, m->state_dev, 8, 0, 0, 1)); // zeros
+    MOON_TRY(alloc_loop(m));
     MOON_TRY(dalloc_t(m, z.H * 8 * 66, &m->attn_partial));
     m->fused = decode_fused_supported(z.d, z.ffn);
     MOON_TRY(dalloc_t(m, z.L * z.H, &m->head_count));
@@ -227,6 +241,8 @@ int alloc_all(moon_text_model *m) {
 
 void free_all(moon_text_model *m) {
     (void)hipStreamSynchronize(m->ctx->stream);
+    layer_list_destroy(m->list);
+    m->list = nullptr;
     for (void *p : m->allocs) (void)hipFree(p);
     m->allocs.clear();
     if (m->ids_pinned) (void)hipHostFree(m->ids_pinned);
@@ -386,6 +402,11 @@ int layer_forward(moon_text_model *m, size_t layer, size_t n, size_t pos, bool p
 
 // lm_head on row `row` of hidden (text_model.zig:325-345)
 int lm_head(moon_text_model *m, size_t row) {
+    if (m->list) {
+        const uint32_t r = (uint32_t)row;
+        size_t ld;
+        return layer_list_logits(m->list, &r, 1, &m->logits_f32, &ld);
+    }
     const Sizes z = sizes(m->cfg);
     ProfScope scope(m, PROF_LM_HEAD);
     if (m->fused)
@@ -393,6 +414,17 @@ int lm_head(moon_text_model *m, size_t row) {
                                      m->logits, z.V, nullptr, nullptr, nullptr, 0);
     MOON_TRY(launch_layernorm(m->ctx, m->hidden + row * z.d, m->lno_w, m->lno_b, m->ln_last, 1, z.d, m->cfg.ln_eps));
     return launch_gemv_nt(m->ctx, m->ln_last, m->lin_w, m->lin_b, m->logits, z.V, z.d, MOON_EPI_BIAS);
+}
+
+// one token through all layers; token_dev, or row 0 of m->hidden
+int step_layers(moon_text_model *m, size_t pos, bool pos_on_device, const uint32_t *token_dev) {
+    if (m->list) return layer_list_step(m->list, token_dev, pos, pos_on_device ? m->state_dev : nullptr);
+    for (size_t l = 0; l < m->cfg.n_layers; l++) MOON_TRY(layer_forward(m, l, 1, pos, pos_on_device, l == 0 ? token_dev : nullptr));
+    return MOON_OK;
+}
+
+int refuse_list(moon_text_model *m, const char *call) {
+    return moon_fail(m->ctx, MOON_EINVAL, "%s: only for the f16 decoder block, not for a decoder opened from a model folder", call);
 }
 
 } // namespace
@@ -529,6 +561,67 @@ extern "C" int moon_text_reset(moon_text_model *m) {
     return MOON_OK;
 }
 
+static int open_list(moon_ctx *ctx, const char *text, size_t len, const SafeTensors *file, int dtype, size_t max_seq, uint64_t seed, float std_dev,
+                     moon_text_model **out) {
+    const Design *design = nullptr;
+    LayerListSpec spec;
+    std::string err;
+    if (int rc = parse_model_config(text, len, &design, &spec, &err); rc != MOON_OK) return moon_fail(ctx, rc, "%s", err.c_str());
+    if (dtype != MOON_DTYPE_BF16 && dtype != MOON_DTYPE_F32) return moon_fail(ctx, MOON_EINVAL, "text_model_open: unknown element type %d", dtype);
+    if (!max_seq || max_seq > 0x3fffffff) return moon_fail(ctx, MOON_EINVAL_DIM, "text_model_open: max_seq %zu", max_seq);
+    MOON_HIP(ctx, hipSetDevice(ctx->device));
+    moon_text_model *m = new moon_text_model();
+    m->ctx = ctx;
+    m->cfg.vocab = spec.vocab;
+    m->cfg.dim = spec.width;
+    m->cfg.n_layers = spec.layers.size();
+    m->cfg.max_seq = max_seq;
+    m->cfg.ln_eps = spec.eps;
+    int rc = alloc_loop(m);
+    if (rc == MOON_OK) rc = layer_list_create(ctx, spec, design, file, seed, std_dev, dtype, max_seq, &m->list);
+    if (rc != MOON_OK) {
+        free_all(m);
+        delete m;
+        return rc;
+    }
+    *out = m;
+    return MOON_OK;
+}
+
+extern "C" int moon_text_model_open(moon_ctx *ctx, const char *dir, int dtype, size_t max_seq, moon_text_model **out) {
+    if (!ctx || !out) return MOON_EINVAL;
+    std::lock_guard<std::mutex> lock(ctx->mu);
+    *out = nullptr;
+    if (!dir) return moon_fail(ctx, MOON_EINVAL, "text_model_open: null folder");
+    const std::string base = std::string(dir) + "/";
+    std::string text, err;
+    FILE *f = fopen((base + "config.json").c_str(), "rb");
+    if (!f) return moon_fail(ctx, MOON_EINVAL, "text_model_open: cannot read %sconfig.json", base.c_str());
+    char buf[4096];
+    for (size_t n; (n = fread(buf, 1, sizeof buf, f)) > 0;) text.append(buf, n);
+    fclose(f);
+    SafeTensors file;
+    if (int rc = file.open(base + "model.safetensors", &err); rc != MOON_OK) return moon_fail(ctx, rc, "%s", err.c_str());
+    return open_list(ctx, text.data(), text.size(), &file, dtype, max_seq, 0, 0.0f, out);
+}
+
+extern "C" int moon_text_model_open_synthetic(moon_ctx *ctx, const char *config_json, int dtype, size_t max_seq, uint64_t seed, float std_dev,
+                                              moon_text_model **out) {
+    if (!ctx || !out) return MOON_EINVAL;
+    std::lock_guard<std::mutex> lock(ctx->mu);
+    *out = nullptr;
+    if (!config_json) return moon_fail(ctx, MOON_EINVAL, "text_model_open_synthetic: null configuration");
+    return open_list(ctx, config_json, strlen(config_json), nullptr, dtype, max_seq, seed, std_dev, out);
+}
+
+extern "C" const char *moon_text_designs(void) {
+    static const std::string names = known_designs();
+    return names.c_str();
+}
+
+extern "C" size_t moon_text_vocab(const moon_text_model *m) { return m ? m->cfg.vocab : 0; }
+extern "C" size_t moon_text_dim(const moon_text_model *m) { return m ? m->cfg.dim : 0; }
+
 extern "C" size_t moon_text_position(const moon_text_model *m) { return m ? m->cur_len : 0; }
 
 // n rows already in m->hidden: the layers, the bookkeeping and, for a single row, the fused kernels' error words
@@ -559,10 +652,66 @@ static int forward_rows_locked(moon_text_model *m, size_t n_ids) {
     return MOON_OK;
 }
 
+// The wanted logits among tokens [lo, lo + n) of the call, which are rows 0 .. n - 1 now, to the caller's memory.
+static int wanted_logits(moon_text_model *m, size_t lo, size_t n, const size_t *want, size_t n_want, float *out) {
+    moon_ctx *ctx = m->ctx;
+    const size_t V = m->cfg.vocab;
+    std::vector<uint32_t> rows;
+    std::vector<size_t> places;
+    for (size_t i = 0; i <= n_want; i++) {
+        if (i < n_want && want[i] >= lo && want[i] < lo + n) {
+            rows.push_back((uint32_t)(want[i] - lo));
+            places.push_back(i);
+        }
+        if (rows.empty() || (i < n_want && rows.size() < (m->list ? LIST_LOGIT_ROWS : 1))) continue;
+        if (m->list) {
+            size_t ld;
+            MOON_TRY(layer_list_logits(m->list, rows.data(), rows.size(), &m->logits_f32, &ld));
+            for (size_t r = 0; r < rows.size(); r++)
+                MOON_HIP(ctx, hipMemcpyAsync(out + places[r] * V, m->logits_f32 + r * ld, V * sizeof(float), hipMemcpyDeviceToHost, ctx->stream));
+            MOON_HIP(ctx, hipStreamSynchronize(ctx->stream));
+        } else {
+            std::vector<half_t> f16(V);
+            MOON_TRY(lm_head(m, rows[0]));
+            MOON_TRY(copy_down_sync(m, f16.data(), m->logits, V * sizeof(half_t)));
+            for (size_t v = 0; v < V; v++) out[places[0] * V + v] = (float)f16[v];
+        }
+        rows.clear();
+        places.clear();
+    }
+    return MOON_OK;
+}
+
+// A list decoder's rows: ids already in ids_pinned, at most layer_list_rows of them at a time (each part attends to the parts
+// before it through the cache, as separate calls would).
+static int forward_list_locked(moon_text_model *m, size_t n_ids, const size_t *want, size_t n_want, float *logits) {
+    moon_ctx *ctx = m->ctx;
+    for (size_t done = 0; done < n_ids;) {
+        const size_t n = std::min(n_ids - done, layer_list_rows(m->list));
+        if (n == 1) MOON_TRY(layer_list_step(m->list, m->ids_dev + done, m->cur_len, nullptr));
+        else MOON_TRY(layer_list_forward(m->list, m->ids_dev + done, n, m->cur_len));
+        m->cur_len += n;
+        m->last_n = n;
+        MOON_TRY(wanted_logits(m, done, n, want, n_want, logits));
+        done += n;
+    }
+    hipLaunchKernelGGL(set_state_kernel, dim3(1), dim3(1), 0, ctx->stream, m->state_dev, (uint32_t)m->cur_len, 0u);
+    MOON_HIP(ctx, hipGetLastError());
+    MOON_HIP(ctx, hipStreamSynchronize(ctx->stream));
+    return MOON_OK;
+}
+
 extern "C" int moon_text_forward(moon_text_model *m, const uint32_t *ids, size_t n_ids) {
+    return moon_text_forward_logits(m, ids, n_ids, nullptr, 0, nullptr);
+}
+
+extern "C" int moon_text_forward_logits(moon_text_model *m, const uint32_t *ids, size_t n_ids, const size_t *want, size_t n_want, float *logits) {
     if (!m) return MOON_EINVAL;
     moon_ctx *ctx = m->ctx;
     std::lock_guard<std::mutex> lock(ctx->mu);
+    if (n_want && (!want || !logits)) return moon_fail(ctx, MOON_EINVAL, "text_forward_logits: null argument");
+    for (size_t i = 0; i < n_want; i++)
+        if (want[i] >= n_ids) return moon_fail(ctx, MOON_EINVAL_DIM, "text_forward_logits: token %zu of %zu", want[i], n_ids);
     if (!ids && n_ids) return moon_fail(ctx, MOON_EINVAL, "text_forward: null ids");
     if (!n_ids) return moon_fail(ctx, MOON_EINVAL_DIM, "text_forward: empty input (InvalidInputShape)");
     if (m->cache_invalid) return moon_fail(ctx, MOON_EHIP, "text_forward: an earlier decode call failed; call moon_text_reset first");
@@ -573,14 +722,17 @@ extern "C" int moon_text_forward(moon_text_model *m, const uint32_t *ids, size_t
     MOON_HIP(ctx, hipSetDevice(ctx->device));
     memcpy(m->ids_pinned, ids, n_ids * sizeof(uint32_t)); // (every call ends with the stream drained: the buffer is free)
     MOON_HIP(ctx, hipMemcpyAsync(m->ids_dev, m->ids_pinned, n_ids * sizeof(uint32_t), hipMemcpyHostToDevice, ctx->stream));
+    if (m->list) return forward_list_locked(m, n_ids, want, n_want, logits);
     MOON_TRY(launch_embed(ctx, m->wte, m->ids_dev, m->hidden, n_ids, m->cfg.dim));
-    return forward_rows_locked(m, n_ids);
+    MOON_TRY(forward_rows_locked(m, n_ids));
+    return wanted_logits(m, 0, n_ids, want, n_want, logits);
 }
 
 extern "C" int moon_text_forward_embeds(moon_text_model *m, const moon_f16 *embeds, size_t n_rows) {
     if (!m) return MOON_EINVAL;
     moon_ctx *ctx = m->ctx;
     std::lock_guard<std::mutex> lock(ctx->mu);
+    if (m->list) return refuse_list(m, "text_forward_embeds");
     if (!embeds && n_rows) return moon_fail(ctx, MOON_EINVAL, "text_forward_embeds: null input");
     if (!n_rows) return moon_fail(ctx, MOON_EINVAL_DIM, "text_forward_embeds: empty input (InvalidInputShape)");
     if (m->cache_invalid) return moon_fail(ctx, MOON_EHIP, "text_forward_embeds: an earlier decode call failed; call moon_text_reset first");
@@ -595,6 +747,7 @@ extern "C" int moon_text_embed(moon_text_model *m, const uint32_t *ids, size_t n
     if (!m) return MOON_EINVAL;
     moon_ctx *ctx = m->ctx;
     std::lock_guard<std::mutex> lock(ctx->mu);
+    if (m->list) return refuse_list(m, "text_embed");
     if ((!ids || !embeds) && n_ids) return moon_fail(ctx, MOON_EINVAL, "text_embed: null argument");
     if (n_ids > m->cfg.max_seq) return moon_fail(ctx, MOON_ESEQ_TOO_LONG, "text_embed: %zu ids > seq_len %zu (SequenceTooLong)", n_ids, m->cfg.max_seq);
     for (size_t i = 0; i < n_ids; i++)
@@ -613,6 +766,7 @@ extern "C" int moon_text_logits(moon_text_model *m, moon_f16 *logits) {
     if (!m) return MOON_EINVAL;
     moon_ctx *ctx = m->ctx;
     std::lock_guard<std::mutex> lock(ctx->mu);
+    if (m->list) return refuse_list(m, "text_logits");
     if (!logits) return moon_fail(ctx, MOON_EINVAL, "text_logits: null output");
     if (!m->last_n) return moon_fail(ctx, MOON_EINVAL, "text_logits: no forward pass yet");
     MOON_HIP(ctx, hipSetDevice(ctx->device));
@@ -624,9 +778,35 @@ extern "C" int moon_text_hidden(moon_text_model *m, moon_f16 *hidden, size_t n_r
     if (!m) return MOON_EINVAL;
     moon_ctx *ctx = m->ctx;
     std::lock_guard<std::mutex> lock(ctx->mu);
+    if (m->list) return refuse_list(m, "text_hidden");
     if (!hidden) return moon_fail(ctx, MOON_EINVAL, "text_hidden: null output");
     if (n_rows > m->last_n) return moon_fail(ctx, MOON_EINVAL_DIM, "text_hidden: %zu rows requested, last forward had %zu", n_rows, m->last_n);
     return copy_down_sync(m, hidden, m->hidden, n_rows * m->cfg.dim * sizeof(moon_f16));
+}
+
+extern "C" int moon_text_logits_f32(moon_text_model *m, float *logits) {
+    if (!m) return MOON_EINVAL;
+    moon_ctx *ctx = m->ctx;
+    std::lock_guard<std::mutex> lock(ctx->mu);
+    if (!logits) return moon_fail(ctx, MOON_EINVAL, "text_logits: null output");
+    if (!m->last_n) return moon_fail(ctx, MOON_EINVAL, "text_logits: no forward pass yet");
+    MOON_HIP(ctx, hipSetDevice(ctx->device));
+    const size_t last = m->last_n - 1;
+    return wanted_logits(m, 0, m->last_n, &last, 1, logits);
+}
+
+extern "C" int moon_text_hidden_f32(moon_text_model *m, float *hidden, size_t n_rows) {
+    if (!m) return MOON_EINVAL;
+    moon_ctx *ctx = m->ctx;
+    std::lock_guard<std::mutex> lock(ctx->mu);
+    if (!hidden) return moon_fail(ctx, MOON_EINVAL, "text_hidden: null output");
+    if (n_rows > m->last_n) return moon_fail(ctx, MOON_EINVAL_DIM, "text_hidden: %zu rows requested, last forward had %zu", n_rows, m->last_n);
+    const size_t n = n_rows * m->cfg.dim;
+    if (m->list) return copy_down_sync(m, hidden, layer_list_hidden(m->list), n * sizeof(float));
+    std::vector<half_t> f16(n);
+    MOON_TRY(copy_down_sync(m, f16.data(), m->hidden, n * sizeof(half_t)));
+    for (size_t i = 0; i < n; i++) hidden[i] = (float)f16[i];
+    return MOON_OK;
 }
 
 // MOON_DECODE_TRACE: where the workgroups of the last whole-layer launch spent their time, by role (microseconds after
@@ -729,11 +909,13 @@ static int greedy_locked(moon_text_model *m, size_t n_steps, uint32_t *out_ids, 
             MOON_TRY(lm_head(m, row));
             ProfScope scope(m, PROF_ARGMAX);
             if (sampling) // u_dev[state[1]] decides; token -> state[2], ids[state[1]++]; the position moves on for every step but the first
-                MOON_TRY(launch_sample(ctx, m->logits, m->cfg.vocab, sampling, 0.f, m->u_dev, state, m->ids_dev, nullptr, step > 0 ? 1u : 0u));
+                MOON_TRY(launch_sample(ctx, m->logits, m->cfg.vocab, sampling, 0.f, m->u_dev, state, m->ids_dev, nullptr, step > 0 ? 1u : 0u,
+                                       m->list ? m->logits_f32 : nullptr));
+            else if (m->list) MOON_TRY(launch_argmax_record_f32(ctx, m->logits_f32, m->cfg.vocab, state, m->ids_dev));
             else
                 MOON_TRY(launch_argmax_record(ctx, m->logits, m->cfg.vocab, state, m->ids_dev)); // token -> state[2], ids[state[1]++]
         }
-        for (size_t l = 0; l < m->cfg.n_layers; l++) MOON_TRY(layer_forward(m, l, 1, m->cur_len + step, true, l == 0 ? state + 2 : nullptr));
+        MOON_TRY(step_layers(m, m->cur_len + step, true, state + 2));
         if (!lm_argmax && !sampling) {
             ProfScope scope(m, PROF_BUMP);
             hipLaunchKernelGGL(bump_pos_kernel, dim3(1), dim3(1), 0, ctx->stream, state);
@@ -848,8 +1030,10 @@ extern "C" int moon_text_next_token(moon_text_model *m, const moon_sampling_conf
     MOON_HIP(ctx, hipSetDevice(ctx->device));
     MOON_TRY(lm_head(m, m->last_n - 1));
     uint32_t *out = m->state_dev + 5; // a word of the loop's state that the loop itself does not use
-    if (!cfg || cfg->method == MOON_SAMPLE_GREEDY) MOON_TRY(launch_argmax(ctx, m->logits, m->cfg.vocab, out));
-    else MOON_TRY(launch_sample(ctx, m->logits, m->cfg.vocab, cfg, u, nullptr, nullptr, nullptr, out));
+    const float *f32 = m->list ? m->logits_f32 : nullptr;
+    if (cfg && cfg->method != MOON_SAMPLE_GREEDY) MOON_TRY(launch_sample(ctx, m->logits, m->cfg.vocab, cfg, u, nullptr, nullptr, nullptr, out, 0, f32));
+    else if (f32) MOON_TRY(launch_argmax_f32(ctx, f32, m->cfg.vocab, out));
+    else MOON_TRY(launch_argmax(ctx, m->logits, m->cfg.vocab, out));
     MOON_HIP(ctx, hipMemcpyAsync(m->host_words + 8, out, sizeof(uint32_t), hipMemcpyDeviceToHost, ctx->stream));
     MOON_HIP(ctx, hipStreamSynchronize(ctx->stream));
     *token = const_cast<volatile uint32_t *>(m->host_words)[8];
@@ -860,6 +1044,7 @@ extern "C" int moon_text_greedy_profile(moon_text_model *m, size_t n_steps, uint
     if (!m) return MOON_EINVAL;
     moon_ctx *ctx = m->ctx;
     std::lock_guard<std::mutex> lock(ctx->mu);
+    if (m->list) return refuse_list(m, "text_greedy_profile");
     if (!avg_us || !launches) return moon_fail(ctx, MOON_EINVAL, "text_greedy_profile: null output");
     if (!m->fused) return moon_fail(ctx, MOON_EINVAL, "text_greedy_profile: only the fused per-layer kernels can be timed per launch");
     StepProfiler prof;
@@ -881,6 +1066,7 @@ extern "C" int moon_text_debug_raise_wait_error(moon_text_model *m) {
     if (!m) return MOON_EINVAL;
     moon_ctx *ctx = m->ctx;
     std::lock_guard<std::mutex> lock(ctx->mu);
+    if (m->list) return refuse_list(m, "text_debug_raise_wait_error");
     const Sizes z = sizes(m->cfg);
     MOON_HIP(ctx, hipSetDevice(ctx->device));
     // the word before each error word is unused (the tail of a counter line, or of the last counter copy): writes {0, 1} to (tail, error word)
@@ -894,6 +1080,7 @@ extern "C" int moon_text_debug_raise_wait_error(moon_text_model *m) {
 extern "C" int moon_text_set_decode_mode(moon_text_model *m, int mode) {
     if (!m) return MOON_EINVAL;
     std::lock_guard<std::mutex> lock(m->ctx->mu);
+    if (m->list) return refuse_list(m, "text_set_decode_mode");
     if (mode != 0 && mode != 2 && mode != 3)
         return moon_fail(m->ctx, MOON_EINVAL, "decode mode must be 0 (one kernel per layer), 2 (three kernels per layer) or 3 (two kernels per layer)");
     m->decode_mode = mode;
@@ -902,6 +1089,7 @@ extern "C" int moon_text_set_decode_mode(moon_text_model *m, int mode) {
 
 extern "C" size_t moon_text_weight_bytes_per_token(const moon_text_model *m) {
     if (!m) return 0;
+    if (m->list) return layer_list_weight_bytes(m->list);
     const Sizes z = sizes(m->cfg);
     const size_t per_layer = 2 * z.d + 3 * z.d * z.d + 3 * z.d + z.d * z.d + z.d + z.ffn * z.d + z.ffn + z.d * z.ffn + z.d;
     return (z.L * per_layer + 2 * z.d + z.V * z.d + z.V) * sizeof(moon_f16);

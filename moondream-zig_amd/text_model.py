@@ -2,6 +2,8 @@
 from __future__ import annotations
 
 import ctypes as C
+import json
+import os
 
 import numpy as np
 
@@ -28,6 +30,9 @@ _SHORT = {"word_token_embedding": "wte", "t_ln_w": "ln_w", "t_ln_b": "ln_b", "t_
           "t_fc2_b": "fc2_b", "t_linear_w": "linear_w", "t_linear_b": "linear_b", "t_ln_out_w": "ln_out_w", "t_ln_out_b": "ln_out_b"}
 
 
+DTYPES = {"bfloat16": L.DTYPE_BF16, "float32": L.DTYPE_F32}
+
+
 class TextModel:
     def __init__(self, cfg: L.TextConfig, weights: dict | None = None, seed: int | None = None, std: float = 0.02,
                  ctx: Context | None = None):
@@ -48,6 +53,29 @@ class TextModel:
         else:
             self.ctx.check(self.ctx.lib.moon_text_model_create_synthetic(self.ctx.handle, C.byref(cfg), seed or 0, std, C.byref(h)))
         self.handle = h
+
+    @classmethod
+    def open(cls, path: str, dtype: str = "bfloat16", max_seq: int = 2048, ctx: Context | None = None) -> "TextModel":
+        """A decoder from a model folder (config.json names a registered design, model.safetensors holds its weights)."""
+        return cls._opened(ctx, lambda c, h: c.lib.moon_text_model_open(c.handle, os.fsencode(path), DTYPES[dtype], max_seq, h), max_seq)
+
+    @classmethod
+    def open_synthetic(cls, config: dict, dtype: str = "bfloat16", max_seq: int = 2048, seed: int = 0, std: float = 0.02,
+                       ctx: Context | None = None) -> "TextModel":
+        """The same with random weights for a configuration."""
+        text = json.dumps(config).encode()
+        return cls._opened(ctx, lambda c, h: c.lib.moon_text_model_open_synthetic(c.handle, text, DTYPES[dtype], max_seq, seed, std, h), max_seq)
+
+    @classmethod
+    def _opened(cls, ctx, call, max_seq):
+        self = cls.__new__(cls)
+        self.handle, self.ctx = None, ctx or default_context()
+        h = C.c_void_p()
+        self.ctx.check(call(self.ctx, C.byref(h)))
+        self.handle = h
+        lib = self.ctx.lib
+        self.cfg = L.TextConfig(vocab=lib.moon_text_vocab(h), dim=lib.moon_text_dim(h), max_seq=max_seq)
+        return self
 
     def close(self):
         if getattr(self, "handle", None) and self.ctx.handle:
@@ -74,6 +102,24 @@ class TextModel:
     def forward(self, ids):
         ids = np.ascontiguousarray(ids, dtype=np.uint32)
         self.ctx.check(self.ctx.lib.moon_text_forward(self.handle, ptr(ids), ids.size))
+
+    def forward_logits(self, ids, want) -> np.ndarray:
+        """forward() that brings back the f32 logits [len(want), vocab] of the given places among ``ids``."""
+        ids = np.ascontiguousarray(ids, dtype=np.uint32)
+        want = np.ascontiguousarray(want, dtype=np.uint64)
+        out = np.empty((want.size, self.cfg.vocab), dtype=np.float32)
+        self.ctx.check(self.ctx.lib.moon_text_forward_logits(self.handle, ptr(ids), ids.size, ptr(want), want.size, ptr(out)))
+        return out
+
+    def logits_f32(self) -> np.ndarray:
+        out = np.empty(self.cfg.vocab, dtype=np.float32)
+        self.ctx.check(self.ctx.lib.moon_text_logits_f32(self.handle, ptr(out)))
+        return out
+
+    def hidden_f32(self, n_rows: int) -> np.ndarray:
+        out = np.empty((n_rows, self.cfg.dim), dtype=np.float32)
+        self.ctx.check(self.ctx.lib.moon_text_hidden_f32(self.handle, ptr(out), n_rows))
+        return out
 
     # ---- the reference's own three calls (text_model.zig:106, 139, 325), for a host that keeps its loop
     def text_encoder(self, ids) -> np.ndarray:
