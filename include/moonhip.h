@@ -283,6 +283,9 @@ int moon_text_model_open(moon_ctx *ctx, const char *dir, int dtype, size_t max_s
  * be a multiple of 64, head sizes of 8. */
 int moon_text_model_open_synthetic(moon_ctx *ctx, const char *config_json, int dtype, size_t max_seq, uint64_t seed, float std_dev,
                                    moon_text_model **out);
+/* Host side only (no device, no context): reads a model folder as moon_text_model_open does and checks that every tensor of the
+ * configuration is there with its shape.  *design (if set) names the design, *n_layers its layers; text of an error in err. */
+int moon_text_folder_check(const char *dir, const char **design, size_t *n_layers, char *err, size_t err_len);
 /* Names of the registered designs, separated by ", ". */
 const char *moon_text_designs(void);
 size_t moon_text_vocab(const moon_text_model *m);

@@ -117,6 +117,7 @@ SIGNATURES = {
     "moon_text_model_create_synthetic": (_i, [_vp, C.POINTER(TextConfig), _u64, _f, _pp]),
     "moon_text_model_open": (_i, [_vp, C.c_char_p, _i, _sz, _pp]),
     "moon_text_model_open_synthetic": (_i, [_vp, C.c_char_p, _i, _sz, _u64, _f, _pp]),
+    "moon_text_folder_check": (_i, [C.c_char_p, C.POINTER(C.c_char_p), C.POINTER(_sz), C.c_char_p, _sz]),
     "moon_text_designs": (C.c_char_p, []),
     "moon_text_vocab": (_sz, [_vp]),
     "moon_text_dim": (_sz, [_vp]),

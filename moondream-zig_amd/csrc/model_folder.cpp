@@ -198,3 +198,103 @@ int parse_model_config(const char *text, size_t len, const Design **design, Laye
     spec->design = (*design)->name;
     return (*design)->parse(c, spec, err) ? MOON_OK : MOON_EFORMAT;
 }
+
+namespace {
+
+int check_tensor(const SafeTensors &file, const std::string &name, std::initializer_list<size_t> shape, std::string *err) {
+    const StTensor *t = file.find(name);
+    if (!t) {
+        *err = "model.safetensors has no tensor '" + name + "'";
+        return MOON_EFORMAT;
+    }
+    if (t->dtype != "BF16" && t->dtype != "F32") {
+        *err = "tensor '" + name + "' is " + t->dtype + ", not BF16 or F32";
+        return MOON_EFORMAT;
+    }
+    if (t->shape != std::vector<size_t>(shape)) {
+        *err = "tensor '" + name + "' does not have the configuration's shape";
+        return MOON_ESHAPE;
+    }
+    return MOON_OK;
+}
+
+} // namespace
+
+// Every tensor of the description, with its shape
+static int check_tensors(const Design &design, const LayerListSpec &s, const SafeTensors &file, std::string *err) {
+    const TensorNames &n = design.names;
+    const size_t w = s.width;
+    int rc = MOON_OK;
+    auto need = [&](const std::string &name, std::initializer_list<size_t> shape) {
+        if (rc == MOON_OK) rc = check_tensor(file, name, shape, err);
+    };
+    need(n.embed(), {s.vocab, w});
+    need(n.head(), {s.vocab, w});
+    need(n.final_norm(), {w});
+    need(n.final_norm() + n.bias_suffix, {w});
+    bool mixing = false;
+    for (size_t i = 0; i < s.layers.size() && rc == MOON_OK; i++) {
+        const MixerSpec &m = s.layers[i].mixer;
+        const FeedForwardSpec &f = s.layers[i].ff;
+        need(n.norm(i), {w});
+        need(n.norm(i) + n.bias_suffix, {w});
+        need(n.mixer(i, "q"), {m.heads * m.dim, w});
+        need(n.mixer(i, "k"), {m.kv_heads * m.dim, w});
+        need(n.mixer(i, "v"), {m.kv_heads * m.vdim, w});
+        need(n.mixer(i, "o"), {w, m.heads * m.vdim});
+        if (m.gate) need(n.mixer(i, "g"), {m.heads * m.vdim, w});
+        if (m.sink) need(n.mixer(i, "sink"), {m.heads});
+        if (m.v_mix && mixing) need(n.mixer(i, "vmix"), {});
+        mixing = mixing || m.v_mix;
+        if (f.kind == FeedForwardSpec::DENSE) {
+            need(n.ff(i, "gate"), {f.ff, w});
+            need(n.ff(i, "up"), {f.ff, w});
+            need(n.ff(i, "down"), {w, f.ff});
+        } else if (f.kind == FeedForwardSpec::EXPERTS) {
+            need(n.ff(i, "router"), {f.experts, w});
+            need(n.ff(i, "correction"), {f.experts});
+            for (size_t e = 0; e < f.experts && rc == MOON_OK; e++) {
+                need(n.expert(i, e, "gate"), {f.ff, w});
+                need(n.expert(i, e, "up"), {f.ff, w});
+                need(n.expert(i, e, "down"), {w, f.ff});
+            }
+        }
+    }
+    return rc;
+}
+
+int read_model_folder(const std::string &dir, const Design **design, LayerListSpec *spec, SafeTensors *file, std::string *err) {
+    const std::string config = dir + "/config.json";
+    FILE *f = fopen(config.c_str(), "rb");
+    if (!f) {
+        *err = "cannot read " + config;
+        return MOON_EINVAL;
+    }
+    std::string text;
+    char buf[4096];
+    for (size_t n; (n = fread(buf, 1, sizeof buf, f)) > 0;) text.append(buf, n);
+    fclose(f);
+    if (int rc = parse_model_config(text.data(), text.size(), design, spec, err); rc != MOON_OK) return rc;
+    if (int rc = file->open(dir + "/model.safetensors", err); rc != MOON_OK) return rc;
+    return check_tensors(**design, *spec, *file, err);
+}
+
+extern "C" int moon_text_folder_check(const char *dir, const char **design, size_t *n_layers, char *err, size_t err_len) {
+    const Design *d = nullptr;
+    LayerListSpec spec;
+    SafeTensors file;
+    std::string text = "null folder";
+    const int rc = dir ? read_model_folder(dir, &d, &spec, &file, &text) : MOON_EINVAL;
+    if (rc != MOON_OK) {
+        if (err && err_len) snprintf(err, err_len, "%s", text.c_str());
+        return rc;
+    }
+    if (design) *design = d->name;
+    if (n_layers) *n_layers = spec.layers.size();
+    return MOON_OK;
+}
+
+extern "C" const char *moon_text_designs(void) {
+    static const std::string names = known_designs();
+    return names.c_str();
+}

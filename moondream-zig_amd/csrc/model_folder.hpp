@@ -46,3 +46,5 @@ std::string known_designs();
 
 // config.json text -> design and description
 int parse_model_config(const char *text, size_t len, const Design **design, LayerListSpec *spec, std::string *err);
+// the whole folder: config.json parsed, the tensor file mapped and checked against it (a MOON_* status)
+int read_model_folder(const std::string &dir, const Design **design, LayerListSpec *spec, SafeTensors *file, std::string *err);

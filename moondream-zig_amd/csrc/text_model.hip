@@ -561,12 +561,8 @@ extern "C" int moon_text_reset(moon_text_model *m) {
     return MOON_OK;
 }
 
-static int open_list(moon_ctx *ctx, const char *text, size_t len, const SafeTensors *file, int dtype, size_t max_seq, uint64_t seed, float std_dev,
-                     moon_text_model **out) {
-    const Design *design = nullptr;
-    LayerListSpec spec;
-    std::string err;
-    if (int rc = parse_model_config(text, len, &design, &spec, &err); rc != MOON_OK) return moon_fail(ctx, rc, "%s", err.c_str());
+static int open_list(moon_ctx *ctx, const LayerListSpec &spec, const Design *design, const SafeTensors *file, int dtype, size_t max_seq, uint64_t seed,
+                     float std_dev, moon_text_model **out) {
     if (dtype != MOON_DTYPE_BF16 && dtype != MOON_DTYPE_F32) return moon_fail(ctx, MOON_EINVAL, "text_model_open: unknown element type %d", dtype);
     if (!max_seq || max_seq > 0x3fffffff) return moon_fail(ctx, MOON_EINVAL_DIM, "text_model_open: max_seq %zu", max_seq);
     MOON_HIP(ctx, hipSetDevice(ctx->device));
@@ -593,16 +589,12 @@ extern "C" int moon_text_model_open(moon_ctx *ctx, const char *dir, int dtype, s
     std::lock_guard<std::mutex> lock(ctx->mu);
     *out = nullptr;
     if (!dir) return moon_fail(ctx, MOON_EINVAL, "text_model_open: null folder");
-    const std::string base = std::string(dir) + "/";
-    std::string text, err;
-    FILE *f = fopen((base + "config.json").c_str(), "rb");
-    if (!f) return moon_fail(ctx, MOON_EINVAL, "text_model_open: cannot read %sconfig.json", base.c_str());
-    char buf[4096];
-    for (size_t n; (n = fread(buf, 1, sizeof buf, f)) > 0;) text.append(buf, n);
-    fclose(f);
+    const Design *design = nullptr;
+    LayerListSpec spec;
     SafeTensors file;
-    if (int rc = file.open(base + "model.safetensors", &err); rc != MOON_OK) return moon_fail(ctx, rc, "%s", err.c_str());
-    return open_list(ctx, text.data(), text.size(), &file, dtype, max_seq, 0, 0.0f, out);
+    std::string err;
+    if (int rc = read_model_folder(dir, &design, &spec, &file, &err); rc != MOON_OK) return moon_fail(ctx, rc, "%s", err.c_str());
+    return open_list(ctx, spec, design, &file, dtype, max_seq, 0, 0.0f, out);
 }
 
 extern "C" int moon_text_model_open_synthetic(moon_ctx *ctx, const char *config_json, int dtype, size_t max_seq, uint64_t seed, float std_dev,
@@ -611,12 +603,11 @@ extern "C" int moon_text_model_open_synthetic(moon_ctx *ctx, const char *config_
     std::lock_guard<std::mutex> lock(ctx->mu);
     *out = nullptr;
     if (!config_json) return moon_fail(ctx, MOON_EINVAL, "text_model_open_synthetic: null configuration");
-    return open_list(ctx, config_json, strlen(config_json), nullptr, dtype, max_seq, seed, std_dev, out);
-}
-
-extern "C" const char *moon_text_designs(void) {
-    static const std::string names = known_designs();
-    return names.c_str();
+    const Design *design = nullptr;
+    LayerListSpec spec;
+    std::string err;
+    if (int rc = parse_model_config(config_json, strlen(config_json), &design, &spec, &err); rc != MOON_OK) return moon_fail(ctx, rc, "%s", err.c_str());
+    return open_list(ctx, spec, design, nullptr, dtype, max_seq, seed, std_dev, out);
 }
 
 extern "C" size_t moon_text_vocab(const moon_text_model *m) { return m ? m->cfg.vocab : 0; }

@@ -2,6 +2,7 @@
 looks up) or the reference's moondream.bin."""
 from __future__ import annotations
 
+import ctypes as C
 import os
 
 from . import _lib as L
@@ -12,6 +13,15 @@ from .context import Context
 def designs() -> list[str]:
     """Designs a model folder may name."""
     return L.load().moon_text_designs().decode().split(", ")
+
+
+def check_folder(path: str) -> tuple[str, int]:
+    """Reads a model folder and checks its tensors against its configuration (no device needed) -> (design, number of layers)."""
+    design, layers, err = C.c_char_p(), C.c_size_t(), C.create_string_buffer(512)
+    rc = L.load().moon_text_folder_check(os.fsencode(path), C.byref(design), C.byref(layers), err, len(err))
+    if rc != L.OK:
+        weights._raise(rc, err)
+    return design.value.decode(), layers.value
 
 
 def open_text_model(path: str, dtype: str | None = None, max_seq: int = 2048, ctx: Context | None = None) -> text_model.TextModel:
