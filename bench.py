@@ -544,6 +544,63 @@ def cpu_baseline(budget_s=5.0):
                        "C restatement of the reference's AVX2 kernels and per-call thread spawning, not the Zig binary")
 
 
+def rikanex_config(width, layers, heads, kv_heads, window, ff=None, experts=None):
+    """A Rikanex decoder with heads of 64 and a dense (ff) or expert (experts, top, ff) feed-forward in every layer."""
+    mlp = dict(kind="dense", ff=ff) if ff else dict(kind="moe", router=dict(experts=experts[0], top=experts[1]), expert=dict(ff=experts[2]))
+    mixer = dict(heads=heads, kv_heads=kv_heads, dim=64, vdim=64, mask=dict(size=window), scale=0.125, v_mix=True)
+    return dict(architecture="Rikanex", vocab=V, width=width, embedding=dict(scale=1.0), norm=dict(eps=1e-5),
+                layers=[dict(type="attention", mixer=mixer, mlp=mlp)] * layers)
+
+
+# name -> (Rikanex configuration, the f16 decoder of equal width, layers, heads and layer bytes).  A layer of the f16 decoder is
+# 4 d^2 + 2 d * hidden weights, one of Rikanex with as many key/value heads 5 d^2 + 3 d * ff.
+RIKANEX_SIZES = {
+    "w2048_l24_dense": (rikanex_config(2048, 24, 32, 32, 1024, ff=4736), dict(dim=2048, hidden_dim=8192, n_layers=24, n_heads=32)),
+    "w2048_l24_dense_grouped": (rikanex_config(2048, 24, 32, 8, 1024, ff=5504), dict(dim=2048, hidden_dim=8192, n_layers=24, n_heads=32)),
+    "w1024_l24_dense": (rikanex_config(1024, 24, 16, 4, 512, ff=2816), dict(dim=1024, hidden_dim=4096, n_layers=24, n_heads=16)),
+    "w2048_l24_experts": (rikanex_config(2048, 24, 32, 8, 1024, experts=(64, 8, 704)), dict(dim=2048, hidden_dim=8192, n_layers=24, n_heads=32)),
+}
+
+
+def time_decoder(ctx, model, prompt, steps, repeats=3):
+    """Median prefill time of `prompt` ids and time per greedily decoded token behind it (wall clock around blocking calls)."""
+    ids = np.random.default_rng(0).integers(0, V, size=prompt).astype(np.uint32)
+    pre, dec = [], []
+    for rep in range(repeats + 1):  # the first round is the warm-up
+        model.reset()
+        ctx.sync()
+        t0 = time.perf_counter()
+        model.forward(ids)
+        ctx.sync()
+        t1 = time.perf_counter()
+        model.greedy(steps)
+        ctx.sync()
+        t2 = time.perf_counter()
+        if rep:
+            pre.append(t1 - t0)
+            dec.append((t2 - t1) / steps)
+    p, d = sorted(pre)[repeats // 2], sorted(dec)[repeats // 2]
+    return dict(prompt=prompt, prefill_ms=p * 1e3, prefill_tokens_per_s=prompt / p, decode_us_per_token=d * 1e6, decode_tokens_per_s=1 / d,
+                weight_bytes_per_token=model.weight_bytes_per_token, weight_gbs=model.weight_bytes_per_token / d / 1e9,
+                weight_frac=model.weight_bytes_per_token / d / 1e9 / HBM_PEAK_GBS)
+
+
+def bench_rikanex(moon, ctx, sizes, prompts=(768, 1920), steps=64):
+    """Prefill and decode of the Rikanex decoder (bf16, random weights) beside the f16 decoder of equal size, in one process."""
+    out = {}
+    for name in sizes:
+        cfg, near = RIKANEX_SIZES[name]
+        m = moon.text_model.TextModel.open_synthetic(cfg, "bfloat16", 2048, seed=0, std=0.02, ctx=ctx)
+        out[name] = {"rikanex": [time_decoder(ctx, m, n, steps) for n in prompts]}
+        m.close()
+        m = moon.text_model.TextModel(moon.text_model.make_config(vocab=V, head_dim=64, max_seq=2048, **near), seed=0, std=0.02, ctx=ctx)
+        out[name]["f16_decoder_one_kernel_per_layer"] = [time_decoder(ctx, m, n, steps) for n in prompts]
+        m.set_decode_mode(2)
+        out[name]["f16_decoder_three_kernels_per_layer"] = [time_decoder(ctx, m, n, steps) for n in prompts]
+        m.close()
+    return out
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -554,6 +611,8 @@ def main():
     ap.add_argument("--only-gemm", action="store_true",
                     help="only the stand-alone GEMM / attention / vision legs, printed as their own JSON line (what a counter run profiles)")
     ap.add_argument("--only-host-loops", action="store_true", help="only the host-stepped and operator-level decode legs")
+    ap.add_argument("--rikanex", nargs="*", metavar="SIZE",
+                    help="only the Rikanex decoder beside the f16 decoder of equal size, as its own JSON line (default: all of %s)" % ", ".join(RIKANEX_SIZES))
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="first run 8 plain 256 MiB copies (copy16_kernel) as the known-traffic yardstick for a counter run")
     ap.add_argument("--decode-mode", type=int, default=None,
@@ -564,6 +623,9 @@ def main():
     if PREFILL + args.warmup + args.steps + PROFILE_STEPS + 2 * SAMPLED_STEPS + 4 > 2048:
         sys.exit("bench.py: prefill 768 + warmup + steps + 32 profiled + 132 further steps must stay within the 2048-token KV cache")
 
+    for name in args.rikanex or []:
+        if name not in RIKANEX_SIZES:
+            sys.exit(f"bench.py: unknown size {name}")
     moon = importlib.import_module("moondream-zig_amd")
     ctx = moon.Context(0)
     if args.calibrate_copy:
@@ -576,6 +638,11 @@ def main():
                "gemm_prefill_fc1": bench_gemm(moon, ctx, 768, 2048, 8192), "gemm_prefill_fc2": bench_gemm(moon, ctx, 768, 8192, 2048),
                "gemm_4096": bench_gemm(moon, ctx, 4096, 4096, 4096, iters=20), "attention": bench_attention(moon, ctx),
                "vision_encoder_27_blocks": bench_vision(moon, ctx)}
+        ctx.close()
+        print(json.dumps(out))
+        return
+    if args.rikanex is not None:
+        out = bench_rikanex(moon, ctx, args.rikanex or list(RIKANEX_SIZES))
         ctx.close()
         print(json.dumps(out))
         return

@@ -2,10 +2,10 @@
 // softmax denominator and an output gate; each of them is an argument.  The cache of a layer is [G][cap][head size]; the keys of
 // position p lie in row p % cap, so a windowed layer needs no more rows than its window and one call's rows together.
 //
-// bf16 runs on the matrix cores.  A 256-thread workgroup is four wavefronts of 32 query rows each: HB heads of one key/value
-// group times 4 / HB row blocks, HB the largest power of two up to 4 that divides the group.  All four walk the same tiles of 64
-// keys, staged in LDS once for the workgroup (the next tile is requested while one is used); a wavefront skips the tiles that
-// none of its rows can see.  Per tile, with v_mfma_f32_32x32x16_bf16 and f32 accumulation,
+// bf16 runs on the matrix cores, arranged like the kernel of attn_prefill.hip: a 256-thread workgroup owns 32 query rows of one
+// head, its four wavefronts take every fourth tile of 64 keys of the range the rows can see, each with an online softmax of its
+// own over private LDS staging, and the four results are merged at the end.  Per tile, with v_mfma_f32_32x32x16_bf16 and f32
+// accumulation,
 //     S^T[key][q] = K . Q^T     (a lane holds 32 scores of ONE query)
 //     O^T[d][q]  += V^T . P^T   (V row-major in LDS, transposed by the LDS load)
 // Scores and weights are f32.  A weight enters the second product as two bf16 terms, its rounding and the remainder, so the
@@ -19,16 +19,21 @@
 
 namespace {
 
-constexpr int WA_KT = 64; // keys per tile
+constexpr int WA_KT = 64, WA_Q = 32, WA_WAVES = 4; // keys per tile, query rows and wavefronts per workgroup
 typedef short wa_short4_t __attribute__((ext_vector_type(4)));
+typedef bf16_t bf16x4_t __attribute__((ext_vector_type(4)));
 
 template <int P> struct WaCfg { // P: head sizes up to P (a multiple of 32), rows zero padded to it
     static constexpr int KSTEPS = P / 16, DT = P / 32, G = P / 8;
     static constexpr int KS = P + 8; // row strides in elements: 128-bit reads of consecutive K rows and the transposing reads of
-    static constexpr int VS = P == 32 ? 32 : P == 64 ? 96 : P + 32 - (P == 96 ? 32 : 0); // 4 consecutive V rows (16 dwords apart mod 64) are conflict free
-    static constexpr int LOADS = WA_KT * G / 256; // 16-byte pieces per thread and operand tile
-    static constexpr size_t LDS_BYTES = size_t(WA_KT) * (KS + VS) * 2;
-    static_assert(WA_KT * G % 256 == 0, "whole pieces");
+    static constexpr int VS = P == 32 ? 32 : P <= 96 ? 96 : P + 32; // 4 consecutive V rows (16 dwords apart mod 64) are conflict free
+    static constexpr int WAVE_ELEMS = WA_KT * (KS > VS ? KS : VS);  // K is only read before the scores, V only after: they share the area
+    static constexpr int LOADS = G;  // 16-byte pieces per lane and operand tile
+    static constexpr bool AHEAD = P <= 128; // the next tile's pieces wait in registers (above, there are too many)
+    static constexpr int SD = P + 4; // merge: O as [wave][q][SD] floats, (m, l) [wave][q] behind them
+    static constexpr size_t TILE_BYTES = size_t(WA_WAVES) * WAVE_ELEMS * 2, MERGE_BYTES = size_t(WA_WAVES) * WA_Q * SD * 4;
+    static constexpr size_t ML_OFFSET = TILE_BYTES > MERGE_BYTES ? TILE_BYTES : MERGE_BYTES;
+    static constexpr size_t LDS_BYTES = ML_OFFSET + 2 * WA_WAVES * WA_Q * 4;
 };
 
 __device__ __forceinline__ wa_short4_t wa_read_tr(const bf16_t *p) {
@@ -36,45 +41,54 @@ __device__ __forceinline__ wa_short4_t wa_read_tr(const bf16_t *p) {
 }
 
 template <int P>
-__global__ __launch_bounds__(256) void window_attn_kernel(WindowAttn p, int HB) {
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2 : 1))) void window_attn_kernel(WindowAttn p) {
     using C = WaCfg<P>;
-    __shared__ __attribute__((aligned(16))) bf16_t lds[C::LDS_BYTES / 2];
-    bf16_t *Ks = lds, *Vs = lds + WA_KT * C::KS;
+    extern __shared__ __attribute__((aligned(16))) bf16_t wa_lds[];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 31, hf = lane >> 5;
-    const int RB = 4 / HB, rows_wg = 32 * RB, n_rb = (p.n + rows_wg - 1) / rows_wg, n_hg = p.H / HB;
-    // a key/value group's row blocks stay on one die where the counts divide; late rows see the most keys: they start first
+    const int n_qb = (p.n + WA_Q - 1) / WA_Q;
+    // Workgroups are dealt to the eight dies round robin: where the count divides, a die takes whole stretches of the (head, block)
+    // list, so heads that share keys and values meet in one L2.  Late blocks see the most keys: they start first.
     int item = blockIdx.x;
-    const int n_items = n_rb * n_hg;
+    const int n_items = n_qb * p.H;
     if (n_items % 8 == 0) item = (item % 8) * (n_items / 8) + item / 8;
-    const int hg = item / n_rb, rb = n_rb - 1 - item % n_rb;
-    const int h = hg * HB + wave % HB, g = h / (p.H / p.G);
-    const int wg_row0 = rb * rows_wg, row0 = wg_row0 + 32 * (wave / HB);
-    const int first_pos = p.pos0 + wg_row0, last_pos = p.pos0 + min(wg_row0 + rows_wg, p.n) - 1;
+    int h = item / n_qb, qb = item % n_qb;
+    if (n_items % 8 == 0 && (n_items / 8) % n_qb == 0) { // whole heads per die: their blocks walk together
+        const int per_die = n_items / 8, heads = per_die / n_qb, j = item % per_die;
+        h = item / per_die * heads + j % heads;
+        qb = j / heads;
+    }
+    qb = n_qb - 1 - qb;
+    const int g = h / (p.H / p.G), row0 = qb * WA_Q;
+    const int first_pos = p.pos0 + row0, last_pos = p.pos0 + min(row0 + WA_Q, p.n) - 1, pos = first_pos + col; // pos: this lane's query
     const int lo_key = p.window ? max(0, first_pos - p.window + 1) : 0;
     const int t_begin = lo_key / WA_KT, t_end = last_pos / WA_KT + 1; // tiles start at multiples of 64 positions
-    const int my_first = p.pos0 + row0, my_last = p.pos0 + min(row0 + 32, p.n) - 1; // (my_last < my_first: no rows)
-    const int my_lo = p.window ? max(0, my_first - p.window + 1) : 0;
-    const int pos = my_first + col; // this lane's query
-    const bf16_t *ck = reinterpret_cast<const bf16_t *>(p.ck) + size_t(g) * p.cap * p.dimp;
-    const bf16_t *cv = reinterpret_cast<const bf16_t *>(p.cv) + size_t(g) * p.cap * p.vdimp;
-    const int kg = p.dimp / 8, vg = p.vdimp / 8;
+    // the head's cache rows as buffers: a 32-bit offset per piece, and what must not be read is an offset past the end (zeros)
+    const int k_bytes = p.cap * p.dimp * 2, v_bytes = p.cap * p.vdimp * 2;
+    const __amdgpu_buffer_rsrc_t kr = __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t *>(reinterpret_cast<const bf16_t *>(p.ck) + size_t(g) * p.cap * p.dimp), 0, k_bytes, 0x00020000);
+    const __amdgpu_buffer_rsrc_t vr = __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t *>(reinterpret_cast<const bf16_t *>(p.cv) + size_t(g) * p.cap * p.vdimp), 0, v_bytes, 0x00020000);
+    bf16_t *Ks = wa_lds + wave * C::WAVE_ELEMS, *Vs = Ks;
 
     lm_u32x4 rk[C::LOADS], rv[C::LOADS];
-    auto load_tile = [&](int t) {
+    auto load = [&](lm_u32x4 (&r)[C::LOADS], const __amdgpu_buffer_rsrc_t rs, int d, int t) {
         const int key0 = t * WA_KT, slot0 = key0 % p.cap;
 #pragma unroll
         for (int i = 0; i < C::LOADS; i++) {
-            const int x = i * 256 + tid, r = x / C::G, c = x % C::G, key = key0 + r;
-            int slot = slot0 + r;
-            if (slot >= p.cap) slot %= p.cap;
-            const bool ok = key >= lo_key && key <= last_pos; // everything else is masked, and may not be there
-            rk[i] = rv[i] = lm_u32x4{0, 0, 0, 0};
-            if (ok && c < kg) rk[i] = *reinterpret_cast<const lm_u32x4 *>(ck + size_t(slot) * p.dimp + c * 8);
-            if (ok && c < vg) rv[i] = *reinterpret_cast<const lm_u32x4 *>(cv + size_t(slot) * p.vdimp + c * 8);
+            const int x = i * 64 + lane, row = x / C::G, c = x % C::G, key = key0 + row;
+            int slot = slot0 + row;
+            if (slot >= p.cap) slot -= p.cap; // (a cache that wraps has more rows than a tile)
+            const int off = key >= lo_key && key <= last_pos && c * 8 < d ? (slot * d + c * 8) * 2 : 0x7fffffff;
+            r[i] = __builtin_bit_cast(lm_u32x4, __builtin_amdgcn_raw_buffer_load_b128(rs, off, 0, 0));
         }
     };
-    load_tile(t_begin);
-
+    auto store = [&](const lm_u32x4 (&r)[C::LOADS], bf16_t *dst, int stride) {
+#pragma unroll
+        for (int i = 0; i < C::LOADS; i++) {
+            const int x = i * 64 + lane;
+            *reinterpret_cast<lm_u32x4 *>(dst + x / C::G * stride + x % C::G * 8) = r[i];
+        }
+    };
+    int t = t_begin + wave;
+    if (C::AHEAD && t < t_end) load(rk, kr, p.dimp, t);
     bf16x8_t qf[C::KSTEPS]; // the MFMA "B" operand: Q[row0 + col][16 s + 8 hf .. + 7]
     {
         const bf16_t *q = reinterpret_cast<const bf16_t *>(p.q) + size_t(min(row0 + col, p.n - 1)) * p.ldq + h * p.dimp;
@@ -85,6 +99,7 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WindowAttn p, int HB) 
             qf[s] = __builtin_bit_cast(bf16x8_t, v);
         }
     }
+    if (C::AHEAD && t < t_end) load(rv, vr, p.vdimp, t);
     int voff[C::DT]; // where this lane points the transposing loads: key 4 hf + (lane % 16) / 4, columns 32 dt + 16 ((lane / 16) % 2) + 4 (lane % 4)
 #pragma unroll
     for (int dt = 0; dt < C::DT; dt++) voff[dt] = (4 * hf + ((lane & 15) >> 2)) * C::VS + 32 * dt + 16 * ((lane >> 4) & 1) + 4 * (lane & 3);
@@ -94,26 +109,18 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WindowAttn p, int HB) 
     for (int dt = 0; dt < C::DT; dt++)
 #pragma unroll
         for (int v = 0; v < 16; v++) o[dt][v] = 0.0f;
-    // the sink is one more score that the denominator has seen before the first key (counted once: in the lower half's sum)
     constexpr float LOG2E = 1.4426950408889634f;
-    float m_run = p.sink ? p.sink[h] * LOG2E : -INFINITY, l_run = p.sink && hf == 0 ? 1.0f : 0.0f;
     const float c2 = p.scale * LOG2E;
+    float m_run = -INFINITY, l_run = 0.0f; // in base-2 units; l_run: this lane's half of the row's sum
 
-    for (int t = t_begin; t < t_end; t++) {
+    for (; t < t_end; t += WA_WAVES) {
         const int key0 = t * WA_KT;
-        __syncthreads(); // the previous tile has been read
-#pragma unroll
-        for (int i = 0; i < C::LOADS; i++) {
-            const int x = i * 256 + tid, r = x / C::G, c = x % C::G;
-            *reinterpret_cast<lm_u32x4 *>(Ks + r * C::KS + c * 8) = rk[i];
-            *reinterpret_cast<lm_u32x4 *>(Vs + r * C::VS + c * 8) = rv[i];
-        }
-        __syncthreads();
-        if (t + 1 < t_end) load_tile(t + 1);
-        if (key0 > my_last || key0 + WA_KT <= my_lo || my_last < my_first) continue; // (the same for the whole wavefront)
-
+        if (!C::AHEAD) load(rk, kr, p.dimp, t);
+        asm volatile("" ::: "memory"); // the V tile of the round before has been read: the K tile takes its place
+        store(rk, Ks, C::KS);
+        if (C::AHEAD && t + WA_WAVES < t_end) load(rk, kr, p.dimp, t + WA_WAVES);
+        if (!C::AHEAD) load(rv, vr, p.vdimp, t);
         float16_t s[2];
-        __builtin_amdgcn_s_setprio(1);
 #pragma unroll
         for (int kt = 0; kt < 2; kt++) {
 #pragma unroll
@@ -123,22 +130,27 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WindowAttn p, int HB) 
                 s[kt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8_t *>(Ks + (32 * kt + col) * C::KS + 16 * st + 8 * hf), qf[st],
                                                                 s[kt], 0, 0, 0);
         }
-        __builtin_amdgcn_s_setprio(0);
         // s[kt][v]: key key0 + 32 kt + 8 (v / 4) + 4 hf + v % 4 against this lane's query
-        const bool edge = key0 + WA_KT - 1 > my_first || (p.window && key0 < my_last - p.window + 1);
         float mx = -INFINITY;
+        if (key0 + WA_KT - 1 > first_pos || (p.window && key0 < last_pos - p.window + 1)) { // some row does not see the whole tile
 #pragma unroll
-        for (int kt = 0; kt < 2; kt++)
+            for (int kt = 0; kt < 2; kt++)
 #pragma unroll
-            for (int v = 0; v < 16; v++) {
-                float x = s[kt][v] * c2;
-                if (edge) {
+                for (int v = 0; v < 16; v++) {
                     const int key = key0 + 32 * kt + 8 * (v >> 2) + 4 * hf + (v & 3);
-                    if (key > pos || (p.window && pos - key >= p.window)) x = -INFINITY;
+                    const float x = key > pos || (p.window && pos - key >= p.window) ? -INFINITY : s[kt][v] * c2;
+                    s[kt][v] = x;
+                    mx = fmaxf(mx, x);
                 }
-                s[kt][v] = x;
-                mx = fmaxf(mx, x);
-            }
+        } else {
+#pragma unroll
+            for (int kt = 0; kt < 2; kt++)
+#pragma unroll
+                for (int v = 0; v < 16; v++) {
+                    s[kt][v] *= c2;
+                    mx = fmaxf(mx, s[kt][v]);
+                }
+        }
         mx = fmaxf(mx, __shfl_xor(mx, 32));
         const float m_new = fmaxf(m_run, mx), m_use = m_new == -INFINITY ? 0.0f : m_new;
         const float alpha = __builtin_amdgcn_exp2f(m_run - m_use);
@@ -157,6 +169,9 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WindowAttn p, int HB) 
         for (int dt = 0; dt < C::DT; dt++)
 #pragma unroll
             for (int v = 0; v < 16; v++) o[dt][v] *= alpha;
+        asm volatile("" ::: "memory"); // the K tile has been read (LDS serves a wavefront in order): V takes its place
+        store(rv, Vs, C::VS);
+        if (C::AHEAD && t + WA_WAVES < t_end) load(rv, vr, p.vdimp, t + WA_WAVES);
         // contraction step (kt, sp) uses the keys a lane holds in s[kt][8 sp .. 8 sp + 7]: key0 + 32 kt + 16 sp + {4 hf + 0..3, 8 + 4 hf + 0..3}
 #pragma unroll
         for (int kt = 0; kt < 2; kt++)
@@ -179,28 +194,51 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WindowAttn p, int HB) 
                 }
             }
     }
-    const int row = row0 + col;
-    const float inv = 1.0f / (l_run + __shfl_xor(l_run, 32));
-    if (row >= p.n) return;
-    const bf16_t *gate = p.gate ? reinterpret_cast<const bf16_t *>(p.gate) + size_t(row) * p.ldq + h * p.vdimp : nullptr;
-    bf16_t *out = reinterpret_cast<bf16_t *>(p.out) + size_t(row) * p.ldo + h * p.vdimp;
-    typedef bf16_t bf16x4_t __attribute__((ext_vector_type(4)));
+
+    // merge the wavefronts' results; the sink is one more term of the denominator
+    const float l_wave = l_run + __shfl_xor(l_run, 32);
+    float *so = reinterpret_cast<float *>(wa_lds), *sm = reinterpret_cast<float *>(reinterpret_cast<char *>(wa_lds) + C::ML_OFFSET), *sl = sm + WA_WAVES * WA_Q;
+    if (hf == 0) {
+        sm[wave * WA_Q + col] = m_run;
+        sl[wave * WA_Q + col] = l_wave;
+    }
+    __syncthreads(); // every wavefront is done with its staging area
+    const float sink = p.sink ? p.sink[h] * LOG2E : -INFINITY;
+    float m_all = sink;
+#pragma unroll
+    for (int w = 0; w < WA_WAVES; w++) m_all = fmaxf(m_all, sm[w * WA_Q + col]);
+    const float f = m_run == -INFINITY ? 0.0f : __builtin_amdgcn_exp2f(m_run - m_all);
 #pragma unroll
     for (int dt = 0; dt < C::DT; dt++)
 #pragma unroll
-        for (int j = 0; j < 4; j++) {
-            const int d = 32 * dt + 8 * j + 4 * hf; // o[dt][4 j .. 4 j + 3] are elements d .. d + 3
-            if (d >= p.vdimp) continue;
-            bf16x4_t r;
-            if (gate) {
-                const bf16x4_t gz = *reinterpret_cast<const bf16x4_t *>(gate + d);
-#pragma unroll
-                for (int e = 0; e < 4; e++) r[e] = (bf16_t)(o[dt][4 * j + e] * inv * lm_sigmoid((float)gz[e]));
-            } else
-#pragma unroll
-                for (int e = 0; e < 4; e++) r[e] = (bf16_t)(o[dt][4 * j + e] * inv);
-            *reinterpret_cast<bf16x4_t *>(out + d) = r;
+        for (int j = 0; j < 4; j++) { // o[dt][4 j .. 4 j + 3] are elements 32 dt + 8 j + 4 hf .. + 3
+            const float4 r = {o[dt][4 * j] * f, o[dt][4 * j + 1] * f, o[dt][4 * j + 2] * f, o[dt][4 * j + 3] * f};
+            *reinterpret_cast<float4 *>(so + (wave * WA_Q + col) * C::SD + 32 * dt + 8 * j + 4 * hf) = r;
         }
+    __syncthreads();
+    const int q = tid & 31, row = row0 + q;
+    if (row >= p.n) return;
+    float l_all = p.sink ? __builtin_amdgcn_exp2f(sink - m_all) : 0.0f;
+#pragma unroll
+    for (int w = 0; w < WA_WAVES; w++) {
+        const float mw = sm[w * WA_Q + q];
+        if (mw != -INFINITY) l_all += __builtin_amdgcn_exp2f(mw - m_all) * sl[w * WA_Q + q];
+    }
+    const float inv = 1.0f / l_all;
+    const bf16_t *gate = p.gate ? reinterpret_cast<const bf16_t *>(p.gate) + size_t(row) * p.ldq + h * p.vdimp : nullptr;
+    bf16_t *out = reinterpret_cast<bf16_t *>(p.out) + size_t(row) * p.ldo + h * p.vdimp;
+    for (int d = (tid >> 5) * 8; d < p.vdimp; d += 64) {
+        float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int w = 0; w < WA_WAVES; w++)
+#pragma unroll
+            for (int e = 0; e < 8; e++) acc[e] += so[(w * WA_Q + q) * C::SD + d + e];
+        bf16x8_t gz = {}, r;
+        if (gate) gz = *reinterpret_cast<const bf16x8_t *>(gate + d);
+#pragma unroll
+        for (int e = 0; e < 8; e++) r[e] = (bf16_t)(acc[e] * inv * (gate ? lm_sigmoid((float)gz[e]) : 1.0f));
+        *reinterpret_cast<bf16x8_t *>(out + d) = r;
+    }
 }
 
 // One wavefront per (row, head): 64 keys at a time, one per lane for the scores, one element per lane for the values.
@@ -255,8 +293,14 @@ __global__ __launch_bounds__(256) void window_attn_rows_kernel(WindowAttn p) {
 }
 
 template <int P> int launch_mfma(moon_ctx *ctx, const WindowAttn &p) {
-    const int per = p.H / p.G, HB = per % 4 == 0 ? 4 : per % 2 == 0 ? 2 : 1, rows_wg = 32 * (4 / HB);
-    hipLaunchKernelGGL(window_attn_kernel<P>, dim3((unsigned)((p.n + rows_wg - 1) / rows_wg * (p.H / HB))), dim3(256), 0, ctx->stream, p, HB);
+    using C = WaCfg<P>;
+    static std::atomic<bool> attr_set[64]; // the opt-in to this much dynamic LDS is per device (and per instantiation)
+    const int dev = ctx->device >= 0 && ctx->device < 64 ? ctx->device : -1;
+    if (dev < 0 || !attr_set[dev].load()) {
+        MOON_HIP(ctx, hipFuncSetAttribute(reinterpret_cast<const void *>(window_attn_kernel<P>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)C::LDS_BYTES));
+        if (dev >= 0) attr_set[dev].store(true);
+    }
+    hipLaunchKernelGGL(window_attn_kernel<P>, dim3((unsigned)((p.n + WA_Q - 1) / WA_Q * p.H)), dim3(256), C::LDS_BYTES, ctx->stream, p);
     MOON_HIP(ctx, hipGetLastError());
     MOON_NOTE_KERNEL(ctx, "window_attn_kernel<%d>", P);
     return MOON_OK;
@@ -271,7 +315,7 @@ int launch_window_attention(moon_ctx *ctx, int dtype, const WindowAttn &p) {
     if ((p.window ? p.window - 1 + p.n : p.pos0 + p.n) > p.cap && p.pos0 + p.n > p.cap)
         return moon_fail(ctx, MOON_EINVAL_DIM, "window attention: %d rows behind a window of %d do not fit %d cache rows", p.n, p.window, p.cap);
     const int big = std::max(p.dimp, p.vdimp);
-    if (dtype == MOON_DTYPE_BF16 && big <= 256) {
+    if (dtype == MOON_DTYPE_BF16 && big <= 256 && size_t(p.cap) * big * 2 < (size_t(1) << 30)) { // (32-bit offsets within a head's rows)
         if (big <= 32) return launch_mfma<32>(ctx, p);
         if (big <= 64) return launch_mfma<64>(ctx, p);
         if (big <= 96) return launch_mfma<96>(ctx, p);

@@ -49,14 +49,27 @@ __global__ __launch_bounds__(1024) void argmax_kernel(const T *__restrict__ logi
     float best = -INFINITY;
     int idx = 0x7fffffff;
     bool any = false;
-    for (int i = threadIdx.x; i < n; i += blockDim.x) {
-        const float v = (float)logits[i];
+    auto look = [&](float v, int i) {
         if (v > best || (!any && v == best)) { // first occurrence within this thread's ascending scan
             best = v;
             idx = i;
             any = true;
         }
+    };
+    constexpr int PER = 16 / (int)sizeof(T), UNROLL = 4; // whole 16-byte pieces first, several requested at a time
+    typedef T piece_t __attribute__((ext_vector_type(PER)));
+    const int pieces = reinterpret_cast<uintptr_t>(logits) % 16 == 0 ? n / PER : 0;
+    for (int g = threadIdx.x; g < pieces; g += UNROLL * blockDim.x) {
+        piece_t v[UNROLL];
+#pragma unroll
+        for (int u = 0; u < UNROLL; u++) v[u] = reinterpret_cast<const piece_t *>(logits)[min(g + u * (int)blockDim.x, pieces - 1)];
+#pragma unroll
+        for (int u = 0; u < UNROLL; u++)
+#pragma unroll
+            for (int e = 0; e < PER; e++)
+                if (g + u * (int)blockDim.x < pieces) look((float)v[u][e], (g + u * (int)blockDim.x) * PER + e);
     }
+    for (int i = pieces * PER + threadIdx.x; i < n; i += blockDim.x) look((float)logits[i], i);
     // reduce (value desc, index asc)
 #pragma unroll
     for (int off = 32; off >= 1; off >>= 1) {

@@ -137,7 +137,7 @@ __device__ __forceinline__ int next_pow2(int v) { return v <= 1 ? 1 : 1 << (32 -
 
 // LDS of an attention workgroup, in floats: q [NH][dimp], new k [dimp], new v [vdimp], scores [NH][keys], reduction [4][NH][vdimp], misc
 __host__ __device__ __forceinline__ size_t mix_lds_floats(int nh, int dimp, int vdimp, int keys) {
-    return size_t(nh) * dimp + dimp + vdimp + size_t(nh) * keys + size_t(4) * nh * vdimp + 4 * nh + 8;
+    return size_t(nh) * dimp + dimp + vdimp + size_t(nh) * keys + size_t(4) * nh * vdimp + 4 * nh + 8; // (launch_decode_mix: at least nh * S before the misc)
 }
 
 // Attention of one token: kv head g, query heads h0 .. h0 + nh - 1, split `split` of S.
@@ -151,6 +151,26 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
     float *s_q = lds, *s_k = s_q + NH * p.dimp, *s_v = s_k + p.dimp, *s_s = s_v + p.vdimp, *s_r = s_s + NH * keys_max, *s_ml = s_r + 4 * NH * p.vdimp;
     T *ck = reinterpret_cast<T *>(p.ck) + size_t(g) * p.cap * p.dimp, *cv = reinterpret_cast<T *>(p.cv) + size_t(g) * p.cap * p.vdimp;
     const bool has_new = cnt > 0 && j1 == pos + 1;
+    // K: lpk lanes per key, V: lpv lanes per key (powers of two); a step is the keys the four wavefronts take at once.  The first
+    // PF steps' rows are requested before anything else: they do not depend on the new token.
+    constexpr int PE = Piece<T>::N, PF = 4;
+    const int kp = p.dimp / PE, lpk = min(64, next_pow2(kp)), kpw = 64 / lpk, sub = lane / lpk, c0 = lane % lpk;
+    const int vp = p.vdimp / PE, lpv = min(64, next_pow2(vp)), vpw = 64 / lpv, vsub = lane / lpv, vc0 = lane % lpv;
+    auto k_piece = [&](int key, int c) { return *reinterpret_cast<const lm_u32x4 *>(ck + size_t(key % p.cap) * p.dimp + c * PE); };
+    auto v_piece = [&](int key, int c) { return *reinterpret_cast<const lm_u32x4 *>(cv + size_t(key % p.cap) * p.vdimp + c * PE); };
+    lm_u32x4 pk[PF], pv[PF];
+#pragma unroll
+    for (int i = 0; i < PF; i++) {
+        const int key = j0 + (i * 4 + wave) * kpw + sub;
+        pk[i] = lm_u32x4{0, 0, 0, 0};
+        if (key < j1 && key != pos && c0 < kp) pk[i] = k_piece(key, c0);
+    }
+#pragma unroll
+    for (int i = 0; i < PF; i++) {
+        const int key = j0 + (i * 4 + wave) * vpw + vsub;
+        pv[i] = lm_u32x4{0, 0, 0, 0};
+        if (key < j1 && key != pos && vc0 < vp) pv[i] = v_piece(key, vc0);
+    }
     for (int task = wave; task < nh + (has_new ? 2 : 0); task += 4) {
         if (task == nh + 1) { // the new value
             const T *first = p.mixes ? reinterpret_cast<const T *>(p.v_first) + (size_t(g) * p.cap_first + pos % p.cap_first) * p.vdimp : nullptr;
@@ -178,34 +198,37 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
         }
     }
     lds_barrier();
-    // scores: LPK lanes per key
-    constexpr int PE = Piece<T>::N;
-    const int kp = p.dimp / PE, lpk = min(64, next_pow2(kp)), kpw = 64 / lpk, sub = lane / lpk, c0 = lane % lpk;
-    for (int j = j0 + wave * kpw; j < j1; j += 4 * kpw) {
-        const int key = j + sub;
+    auto score_step = [&](int key, const lm_u32x4 &first) {
         float acc[NH];
 #pragma unroll
         for (int h = 0; h < NH; h++) acc[h] = 0.0f;
-        if (key < j1) {
-            const T *kr = ck + size_t(key % p.cap) * p.dimp;
+        if (key < j1)
             for (int c = c0; c < kp; c += lpk) {
                 float kf[PE];
                 if (key == pos) {
 #pragma unroll
                     for (int e = 0; e < PE; e++) kf[e] = s_k[c * PE + e];
-                } else Piece<T>::unpack(*reinterpret_cast<const lm_u32x4 *>(kr + c * PE), kf);
+                } else Piece<T>::unpack(c == c0 ? first : k_piece(key, c), kf);
 #pragma unroll
                 for (int h = 0; h < NH; h++)
                     if (h < nh)
 #pragma unroll
                         for (int e = 0; e < PE; e++) acc[h] = fmaf(kf[e], s_q[h * p.dimp + c * PE + e], acc[h]);
             }
-        }
 #pragma unroll
         for (int h = 0; h < NH; h++) {
             for (int off = lpk >> 1; off >= 1; off >>= 1) acc[h] += __shfl_xor(acc[h], off);
             if (key < j1 && c0 == 0 && h < nh) s_s[h * keys_max + key - j0] = acc[h] * p.scale;
         }
+    };
+#pragma unroll
+    for (int i = 0; i < PF; i++)
+        if (j0 + (i * 4 + wave) * kpw < j1) score_step(j0 + (i * 4 + wave) * kpw + sub, pk[i]);
+    for (int j = j0 + (PF * 4 + wave) * kpw; j < j1; j += 4 * kpw) {
+        const int key = j + sub;
+        lm_u32x4 first = {0, 0, 0, 0};
+        if (key < j1 && key != pos && c0 < kp) first = k_piece(key, c0);
+        score_step(key, first);
     }
     lds_barrier();
     for (int h = wave; h < nh; h += 4) {
@@ -225,30 +248,34 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
         }
     }
     lds_barrier();
-    // values: LPV lanes per key
-    const int vp = p.vdimp / PE, lpv = min(64, next_pow2(vp)), vpw = 64 / lpv, vsub = lane / lpv, vc0 = lane % lpv;
     for (int c = vc0; c < (vp + lpv - 1) / lpv * lpv; c += lpv) {
         float acc[NH][PE];
 #pragma unroll
         for (int h = 0; h < NH; h++)
 #pragma unroll
             for (int e = 0; e < PE; e++) acc[h][e] = 0.0f;
-        if (c < vp)
-            for (int i = wave * vpw + vsub; i < cnt; i += 4 * vpw) {
-                const int key = j0 + i;
-                float vf[PE];
-                if (key == pos) {
+        auto value_step = [&](int key, const lm_u32x4 &piece) {
+            float vf[PE];
+            if (key == pos) {
 #pragma unroll
-                    for (int e = 0; e < PE; e++) vf[e] = s_v[c * PE + e];
-                } else Piece<T>::unpack(*reinterpret_cast<const lm_u32x4 *>(cv + size_t(key % p.cap) * p.vdimp + c * PE), vf);
+                for (int e = 0; e < PE; e++) vf[e] = s_v[c * PE + e];
+            } else Piece<T>::unpack(piece, vf);
 #pragma unroll
-                for (int h = 0; h < NH; h++)
-                    if (h < nh) {
-                        const float w = s_s[h * keys_max + i];
+            for (int h = 0; h < NH; h++)
+                if (h < nh) {
+                    const float w = s_s[h * keys_max + key - j0];
 #pragma unroll
-                        for (int e = 0; e < PE; e++) acc[h][e] = fmaf(w, vf[e], acc[h][e]);
-                    }
+                    for (int e = 0; e < PE; e++) acc[h][e] = fmaf(w, vf[e], acc[h][e]);
+                }
+        };
+        if (c < vp) {
+#pragma unroll
+            for (int i = 0; i < PF; i++) {
+                const int key = j0 + (i * 4 + wave) * vpw + vsub;
+                if (key < j1) value_step(key, c == vc0 || key == pos ? pv[i] : v_piece(key, c));
             }
+            for (int key = j0 + (PF * 4 + wave) * vpw + vsub; key < j1; key += 4 * vpw) value_step(key, key == pos ? pv[0] : v_piece(key, c));
+        }
 #pragma unroll
         for (int h = 0; h < NH; h++)
 #pragma unroll
@@ -278,19 +305,36 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
     }
     __syncthreads();
     if (!*s_last) return;
+    // All of a head's splits: the weight of each (a lane per split) to LDS, then the sums with several loads in flight.
+    float *s_w = lds; // [nh][S], over what the phases before have used
+    for (int h = wave; h < nh; h += 4) {
+        const float *ph = part + size_t(h) * stride + p.vdimp, sink = p.sink ? p.sink[h0 + h] : -INFINITY;
+        float m = sink, l = 0.0f;
+        for (int s = lane; s < S; s += 64) m = fmaxf(m, ld_f<true>(ph + size_t(s) * MIX_HEADS * stride));
+        m = wave_max(m);
+        for (int s = lane; s < S; s += 64) {
+            const float w = expf(ld_f<true>(ph + size_t(s) * MIX_HEADS * stride) - m); // (an empty split: m = -inf, weight 0)
+            l = fmaf(ld_f<true>(ph + size_t(s) * MIX_HEADS * stride + 1), w, l);
+            s_w[h * S + s] = w;
+        }
+        l = wave_sum(l) + (p.sink ? expf(sink - m) : 0.0f);
+        if (lane == 0) s_ml[h] = 1.0f / l;
+    }
+    lds_barrier();
     for (int i = tid; i < nh * p.vdimp; i += 256) {
         const int h = i / p.vdimp, d = i % p.vdimp;
-        const float *ph = part + size_t(h) * stride;
-        float m = p.sink ? p.sink[h0 + h] : -INFINITY;
-        for (int s = 0; s < S; s++) m = fmaxf(m, ld_f<true>(ph + size_t(s) * MIX_HEADS * stride + p.vdimp));
-        float l = p.sink ? expf(p.sink[h0 + h] - m) : 0.0f, o = 0.0f;
-        for (int s = 0; s < S; s++) {
-            const float *ps = ph + size_t(s) * MIX_HEADS * stride;
-            const float w = expf(ld_f<true>(ps + p.vdimp) - m); // (an empty split: m = -inf, weight 0)
-            l = fmaf(ld_f<true>(ps + p.vdimp + 1), w, l);
-            o = fmaf(ld_f<true>(ps + d), w, o);
+        const float *ph = part + size_t(h) * stride + d;
+        constexpr int AT_ONCE = 8;
+        float o = 0.0f;
+        for (int s0 = 0; s0 < S; s0 += AT_ONCE) {
+            float v[AT_ONCE];
+#pragma unroll
+            for (int u = 0; u < AT_ONCE; u++) v[u] = ld_f<true>(ph + size_t(min(s0 + u, S - 1)) * MIX_HEADS * stride);
+#pragma unroll
+            for (int u = 0; u < AT_ONCE; u++)
+                if (s0 + u < S) o = fmaf(v[u], s_w[h * S + s0 + u], o);
         }
-        o /= l;
+        o *= s_ml[h];
         if (p.gate) o *= lm_sigmoid(p.proj[p.og + (h0 + h) * p.vdimp + d]);
         reinterpret_cast<T *>(p.out)[(h0 + h) * p.vdimp + d] = (T)o;
     }
@@ -417,7 +461,7 @@ template <class T, int NH> int mix_launch(moon_ctx *ctx, const DecodeMix &p, int
 template <class T> int proj_launch(moon_ctx *ctx, const DecodeProj &p) {
     const int cus = ctx->cu_count > 0 ? ctx->cu_count : 256;
     const int groups = (p.n16_used + 3) / 4 + (p.n32_used + 3) / 4 + (p.ff + 1) / 2;
-    const dim3 grid((unsigned)std::max(1, std::min(2 * cus, (groups + 3) / 4)));
+    const dim3 grid((unsigned)std::max(1, std::min(4 * cus, (groups + 3) / 4)));
     const size_t lds = size_t(p.dp) * sizeof(T) + size_t(p.width) * sizeof(float);
     const int ch = (p.dp / Piece<T>::N + 63) / 64;
     auto kern = ch == 1 ? decode_proj_kernel<T, 1> : ch == 2 ? decode_proj_kernel<T, 2> : ch == 3 ? decode_proj_kernel<T, 3> : decode_proj_kernel<T, 4>;
@@ -466,6 +510,7 @@ int launch_decode_mix(moon_ctx *ctx, int dtype, const DecodeMix &p) {
     const size_t el = dtype == MOON_DTYPE_BF16 ? sizeof(bf16_t) : sizeof(float);
     const size_t lds = std::max(mix_lds_floats(NH, p.dimp, p.vdimp, keys_max) * sizeof(float),
                                 p.E ? size_t(p.dp) * el + (size_t(2) * p.E + 2 * p.top) * sizeof(float) : 0);
+    if (size_t(NH) * S > mix_lds_floats(NH, p.dimp, p.vdimp, keys_max) - 4 * NH - 8) return moon_fail(ctx, MOON_ESEQ_TOO_LONG, "decode attention: %d splits", S);
     if (lds > 160 * 1024) return moon_fail(ctx, MOON_EINVAL_DIM, "decode attention: heads of %d and %d", p.dimp, p.vdimp);
     auto go = [&](auto tag) -> int {
         using T = decltype(tag);

@@ -17,8 +17,8 @@ struct LayerList {
     int first_mix = -1;
     void *embed = nullptr, *head = nullptr;
     float *fgamma = nullptr, *fbeta = nullptr;
-    float *x = nullptr, *router = nullptr, *partial = nullptr, *proj = nullptr, *y = nullptr, *logits = nullptr, *mix_partial = nullptr, *weight = nullptr;
-    void *h = nullptr, *c1 = nullptr, *a2 = nullptr, *act = nullptr;
+    float *x = nullptr, *router = nullptr, *partial = nullptr, *proj = nullptr, *logits = nullptr, *mix_partial = nullptr, *weight = nullptr;
+    void *h = nullptr, *c1 = nullptr, *a2 = nullptr, *act = nullptr, *y = nullptr;
     int *ids = nullptr, *slot = nullptr, *tile_group = nullptr, *tile_row = nullptr, *tile_end = nullptr, *n_tiles = nullptr;
     uint32_t *grouped_rows = nullptr, *counter = nullptr, *want = nullptr;
     uint32_t *want_pinned = nullptr;
@@ -265,7 +265,7 @@ int create(LayerList *l, const Design *design, const SafeTensors *file, uint64_t
     MOON_TRY(alloc_n(l, n16, &l->proj));
     MOON_TRY(alloc_n(l, std::max(R, std::min(8 * R, 128 * cus / tiles_n)) * l->dp, &l->partial)); // (see seg_gemm_splits)
     MOON_TRY(alloc_t(l, act, &l->act));
-    MOON_TRY(alloc_n(l, y, &l->y));
+    MOON_TRY(alloc_t(l, y, &l->y));
     MOON_TRY(alloc_n(l, pairs, &l->ids));
     MOON_TRY(alloc_n(l, pairs, &l->slot));
     MOON_TRY(alloc_n(l, pairs, &l->weight));
@@ -442,11 +442,11 @@ int layer_list_forward(LayerList *l, const uint32_t *ids_dev, size_t n_rows, siz
             e.rows = nullptr;
             e.W = d.wd;
             e.w_group = size_t(dp) * d.ffp;
-            e.N = e.n32 = dp;
+            e.N = e.n16 = e.n32 = dp;
             e.K = d.ffp;
             e.glu = nullptr;
-            e.c32 = l->y;
-            e.ld32 = dp;
+            e.c16 = l->y;
+            e.ld16 = dp;
             MOON_TRY(launch_seg_gemm(ctx, dt, e));
             f.expert_out = l->y;
             f.slot = l->slot;

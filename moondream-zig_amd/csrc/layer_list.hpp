@@ -93,7 +93,7 @@ struct RowFinish {
     float embed_scale;
     const float *partial;     // [splits][n][dp]
     int splits;
-    const float *expert_out;  // [n * top][dp], rows in the order of `slot`
+    const void *expert_out;   // T [n * top][dp], rows in the order of `slot`
     const int *slot;          // [n][top]
     const float *weight;      // [n][top]
     int top;

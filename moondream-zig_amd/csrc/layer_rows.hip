@@ -5,71 +5,142 @@
 #include "norm.hpp"
 #include "router.hpp"
 
+#include <algorithm>
+
 namespace {
 
-template <class T>
+template <class T, int W> struct RowVec; // W consecutive elements
+template <class T> struct RowVec<T, 1> {
+    static __device__ __forceinline__ void load(const T *p, float (&v)[1]) { v[0] = (float)p[0]; }
+    static __device__ __forceinline__ void store(T *p, const float (&v)[1]) { p[0] = (T)v[0]; }
+};
+template <class T> struct RowVec<T, 4> {
+    typedef T vec __attribute__((ext_vector_type(4)));
+    static __device__ __forceinline__ void load(const T *p, float (&v)[4]) {
+        const vec x = *reinterpret_cast<const vec *>(p);
+#pragma unroll
+        for (int e = 0; e < 4; e++) v[e] = (float)x[e];
+    }
+    static __device__ __forceinline__ void store(T *p, const float (&v)[4]) {
+        vec x;
+#pragma unroll
+        for (int e = 0; e < 4; e++) x[e] = (T)v[e];
+        *reinterpret_cast<vec *>(p) = x;
+    }
+};
+
+// W: elements a thread takes at a time (4 where the width allows)
+template <class T, int W>
 __global__ __launch_bounds__(256) void row_finish_kernel(RowFinish p) {
     extern __shared__ __attribute__((aligned(16))) float s_row[]; // [width]
     __shared__ float sm[16];
     const int r = blockIdx.x, tid = threadIdx.x;
     float *xr = p.x + size_t(p.rows ? p.rows[r] : (uint32_t)r) * p.width;
     const T *er = p.embed ? reinterpret_cast<const T *>(p.embed) + size_t(p.ids[r]) * p.dp : nullptr;
+    const T *eo = reinterpret_cast<const T *>(p.expert_out);
     const bool changes = er || p.splits || p.top;
     float s = 0.0f;
-    for (int i = tid; i < p.width; i += 256) {
-        float v;
-        if (er) v = (float)er[i] * p.embed_scale;
-        else {
-            float d = 0.0f;
-            for (int k = 0; k < p.splits; k++) d += p.partial[(size_t(k) * p.n + r) * p.dp + i];
-            for (int k = 0; k < p.top; k++) d = fmaf(p.weight[r * p.top + k], p.expert_out[size_t(p.slot[r * p.top + k]) * p.dp + i], d);
-            v = xr[i] + d;
+    for (int i = tid * W; i < p.width; i += 256 * W) {
+        float v[W], d[W] = {};
+        if (er) {
+            RowVec<T, W>::load(er + i, v);
+#pragma unroll
+            for (int e = 0; e < W; e++) v[e] *= p.embed_scale;
+        } else {
+            RowVec<float, W>::load(xr + i, v);
+#pragma unroll 4
+            for (int k = 0; k < p.splits; k++) {
+                float t[W];
+                RowVec<float, W>::load(p.partial + (size_t(k) * p.n + r) * p.dp + i, t);
+#pragma unroll
+                for (int e = 0; e < W; e++) d[e] += t[e];
+            }
+#pragma unroll 4
+            for (int k = 0; k < p.top; k++) {
+                float t[W];
+                RowVec<T, W>::load(eo + size_t(p.slot[r * p.top + k]) * p.dp + i, t);
+                const float w = p.weight[r * p.top + k];
+#pragma unroll
+                for (int e = 0; e < W; e++) d[e] = fmaf(w, t[e], d[e]);
+            }
+#pragma unroll
+            for (int e = 0; e < W; e++) v[e] += d[e];
         }
-        if (changes) xr[i] = v;
-        s_row[i] = v;
-        s += v;
+        if (changes) RowVec<float, W>::store(xr + i, v);
+        RowVec<float, W>::store(s_row + i, v);
+#pragma unroll
+        for (int e = 0; e < W; e++) s += v[e];
     }
     if (!p.h) return;
     const float mean = block_sum(s, sm) / (float)p.width;
     float m2 = 0.0f;
-    for (int i = tid; i < p.width; i += 256) { // (each thread reads back what it wrote)
-        const float d = s_row[i] - mean;
-        m2 = fmaf(d, d, m2);
-    }
+    for (int i = tid * W; i < p.width; i += 256 * W) // (each thread reads back what it wrote)
+#pragma unroll
+        for (int e = 0; e < W; e++) {
+            const float d = s_row[i + e] - mean;
+            m2 = fmaf(d, d, m2);
+        }
     const float rstd = 1.0f / sqrtf(block_sum(m2, sm) / (float)p.width + p.eps);
     T *h = reinterpret_cast<T *>(p.h) + size_t(r) * p.dp;
-    for (int i = tid; i < p.dp; i += 256) h[i] = i < p.width ? (T)((s_row[i] - mean) * rstd * p.gamma[i] + p.beta[i]) : (T)0.0f;
+    for (int i = tid * W; i < p.dp; i += 256 * W) {
+        float v[W] = {}, ga[W], be[W];
+        if (i < p.width) {
+            RowVec<float, W>::load(p.gamma + i, ga);
+            RowVec<float, W>::load(p.beta + i, be);
+#pragma unroll
+            for (int e = 0; e < W; e++) v[e] = (s_row[i + e] - mean) * rstd * ga[e] + be[e];
+        }
+        RowVec<T, W>::store(h + i, v);
+    }
 }
 
+// lph lanes (a power of two) per head of a row; a workgroup's heads follow each other in (row, head) order.
 template <class T>
-__global__ __launch_bounds__(256) void prep_qkv_kernel(PrepArgs p) {
-    const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+__global__ __launch_bounds__(256) void prep_qkv_kernel(PrepArgs p, int lph) {
+    constexpr int PE = Piece<T>::N;
+    const int tasks = p.H + 2 * p.G, at = (int)(blockIdx.x * 256 + threadIdx.x) / lph, c0 = threadIdx.x % lph;
+    const int r = at / tasks, task = at % tasks;
+    if (r >= p.n) return; // (whole groups of lph lanes)
     T *row = reinterpret_cast<T *>(p.c1) + size_t(r) * p.ld;
     const int pos = p.pos0 + r, slot = pos % p.cap;
-    for (int task = blockIdx.y * 4 + wave; task < p.H + 2 * p.G; task += gridDim.y * 4) {
-        if (task < p.H + p.G) { // a head of q or k
-            const bool is_q = task < p.H;
-            const int g = task - p.H;
-            T *src = row + (is_q ? p.oq + task * p.dimp : p.ok + g * p.dimp);
-            T *dst = is_q ? src : reinterpret_cast<T *>(p.ck) + (size_t(g) * p.cap + slot) * p.dimp;
-            if (is_q && !p.qk_rms) continue;
-            float ss = 0.0f;
-            for (int d = lane; d < p.dimp; d += 64) { // (the padding is zero)
-                const float v = (float)src[d];
-                ss = fmaf(v, v, ss);
+    if (task < p.H + p.G) { // a head of q or k
+        const bool is_q = task < p.H;
+        if (is_q && !p.qk_rms) return;
+        const int g = task - p.H, pieces = p.dimp / PE;
+        T *src = row + (is_q ? p.oq + task * p.dimp : p.ok + g * p.dimp);
+        T *dst = is_q ? src : reinterpret_cast<T *>(p.ck) + (size_t(g) * p.cap + slot) * p.dimp;
+        float ss = 0.0f, v[PE];
+        for (int c = c0; c < pieces; c += lph) { // (the padding is zero)
+            Piece<T>::unpack(*reinterpret_cast<const lm_u32x4 *>(src + c * PE), v);
+#pragma unroll
+            for (int e = 0; e < PE; e++) ss = fmaf(v[e], v[e], ss);
+        }
+        for (int off = lph >> 1; off >= 1; off >>= 1) ss += __shfl_xor(ss, off);
+        const float f = p.qk_rms ? 1.0f / sqrtf(ss / (float)p.dim + p.eps) : 1.0f;
+        for (int c = c0; c < pieces; c += lph) {
+            Piece<T>::unpack(*reinterpret_cast<const lm_u32x4 *>(src + c * PE), v);
+            lm_u32x4 o;
+            T *t = reinterpret_cast<T *>(&o);
+#pragma unroll
+            for (int e = 0; e < PE; e++) t[e] = (T)(v[e] * f);
+            *reinterpret_cast<lm_u32x4 *>(dst + c * PE) = o;
+        }
+    } else {
+        const int g = task - p.H - p.G, pieces = p.vdimp / PE;
+        const T *src = row + p.ov + g * p.vdimp;
+        T *dst = reinterpret_cast<T *>(p.cv) + (size_t(g) * p.cap + slot) * p.vdimp;
+        const T *first = p.mixes ? reinterpret_cast<const T *>(p.v_first) + (size_t(g) * p.cap_first + pos % p.cap_first) * p.vdimp : nullptr;
+        for (int c = c0; c < pieces; c += lph) {
+            float v[PE], f[PE];
+            lm_u32x4 o = *reinterpret_cast<const lm_u32x4 *>(src + c * PE);
+            if (first) {
+                Piece<T>::unpack(o, v);
+                Piece<T>::unpack(*reinterpret_cast<const lm_u32x4 *>(first + c * PE), f);
+                T *t = reinterpret_cast<T *>(&o);
+#pragma unroll
+                for (int e = 0; e < PE; e++) t[e] = (T)((1.0f - p.lambda) * v[e] + p.lambda * f[e]);
             }
-            const float f = p.qk_rms ? 1.0f / sqrtf(wave_sum(ss) / (float)p.dim + p.eps) : 1.0f;
-            for (int d = lane; d < p.dimp; d += 64) dst[d] = (T)((float)src[d] * f);
-        } else {
-            const int g = task - p.H - p.G;
-            const T *src = row + p.ov + g * p.vdimp;
-            T *dst = reinterpret_cast<T *>(p.cv) + (size_t(g) * p.cap + slot) * p.vdimp;
-            const T *first = p.mixes ? reinterpret_cast<const T *>(p.v_first) + (size_t(g) * p.cap_first + pos % p.cap_first) * p.vdimp : nullptr;
-            for (int d = lane; d < p.vdimp; d += 64) {
-                float v = (float)src[d];
-                if (first) v = (1.0f - p.lambda) * v + p.lambda * (float)first[d];
-                dst[d] = (T)v;
-            }
+            *reinterpret_cast<lm_u32x4 *>(dst + c * PE) = o;
         }
     }
 }
@@ -125,12 +196,12 @@ __global__ __launch_bounds__(1024) void group_kernel(RouteArgs p) {
     for (int base = lo; base < hi; base += 64) { // 64 pairs at a time, in order
         const int i = base + lane;
         const int e = i < hi ? p.ids[i] : -1;
-        int before = 0, same = 0;
-        for (int l = 0; l < 64; l++) {
-            const int other = __shfl(e, l);
-            before += other == e && l < lane ? 1 : 0;
-            same += other == e ? 1 : 0;
+        unsigned long long match = ~0ull; // the lanes with this lane's expert
+        for (int bit = 1; bit < 2 * p.E; bit <<= 1) { // (lanes past the end count as expert E)
+            const unsigned long long ones = __ballot(((e < 0 ? p.E : e) & bit) != 0);
+            match &= (e < 0 ? p.E : e) & bit ? ones : ~ones;
         }
+        const int before = __popcll(match & ((1ull << lane) - 1)), same = __popcll(match);
         if (e >= 0) {
             const int at = per_wave[wave * p.E + e] + before;
             p.slot[i] = at;
@@ -148,8 +219,9 @@ int launch_row_finish(moon_ctx *ctx, int dtype, const RowFinish &p) {
     if (p.n <= 0) return MOON_OK;
     const size_t lds = size_t(p.width) * sizeof(float);
     if (lds > 60 * 1024) return moon_fail(ctx, MOON_EINVAL_DIM, "row kernel: width %d too large", p.width);
-    if (dtype == MOON_DTYPE_BF16) hipLaunchKernelGGL(row_finish_kernel<bf16_t>, dim3(p.n), dim3(256), lds, ctx->stream, p);
-    else hipLaunchKernelGGL(row_finish_kernel<float>, dim3(p.n), dim3(256), lds, ctx->stream, p);
+    auto kern = dtype == MOON_DTYPE_BF16 ? (p.width % 4 ? row_finish_kernel<bf16_t, 1> : row_finish_kernel<bf16_t, 4>)
+                                         : (p.width % 4 ? row_finish_kernel<float, 1> : row_finish_kernel<float, 4>);
+    hipLaunchKernelGGL(kern, dim3(p.n), dim3(256), lds, ctx->stream, p);
     MOON_HIP(ctx, hipGetLastError());
     return MOON_OK;
 }
@@ -157,9 +229,12 @@ int launch_row_finish(moon_ctx *ctx, int dtype, const RowFinish &p) {
 int launch_prep_qkv(moon_ctx *ctx, int dtype, const PrepArgs &p) {
     if (p.n <= 0) return MOON_OK;
     if (p.n > p.cap || (p.mixes && p.n > p.cap_first)) return moon_fail(ctx, MOON_EINVAL_DIM, "cache update: %d rows, %d slots", p.n, p.cap);
-    const dim3 grid(p.n, p.n < 512 ? (unsigned)((p.H + 2 * p.G + 3) / 4) : 1);
-    if (dtype == MOON_DTYPE_BF16) hipLaunchKernelGGL(prep_qkv_kernel<bf16_t>, grid, dim3(256), 0, ctx->stream, p);
-    else hipLaunchKernelGGL(prep_qkv_kernel<float>, grid, dim3(256), 0, ctx->stream, p);
+    const int pieces = std::max(p.dimp, p.vdimp) / (dtype == MOON_DTYPE_BF16 ? Piece<bf16_t>::N : Piece<float>::N);
+    int lph = 1;
+    while (lph < pieces && lph < 64) lph *= 2;
+    const dim3 grid((unsigned)((size_t(p.n) * (p.H + 2 * p.G) * lph + 255) / 256));
+    if (dtype == MOON_DTYPE_BF16) hipLaunchKernelGGL(prep_qkv_kernel<bf16_t>, grid, dim3(256), 0, ctx->stream, p, lph);
+    else hipLaunchKernelGGL(prep_qkv_kernel<float>, grid, dim3(256), 0, ctx->stream, p, lph);
     MOON_HIP(ctx, hipGetLastError());
     return MOON_OK;
 }
