@@ -21,7 +21,8 @@ namespace {
 
 constexpr int WA_KT = 64, WA_Q = 32, WA_WAVES = 4; // keys per tile, query rows and wavefronts per workgroup
 typedef short wa_short4_t __attribute__((ext_vector_type(4)));
-typedef bf16_t bf16x4_t __attribute__((ext_vector_type(4)));
+typedef bf16_t bf16x2_t __attribute__((ext_vector_type(2)));
+typedef float float2_t __attribute__((ext_vector_type(2)));
 
 template <int P> struct WaCfg { // P: head sizes up to P (a multiple of 32), rows zero padded to it
     static constexpr int KSTEPS = P / 16, DT = P / 32, G = P / 8;
@@ -68,16 +69,29 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
     const __amdgpu_buffer_rsrc_t vr = __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t *>(reinterpret_cast<const bf16_t *>(p.cv) + size_t(g) * p.cap * p.vdimp), 0, v_bytes, 0x00020000);
     bf16_t *Ks = wa_lds + wave * C::WAVE_ELEMS, *Vs = Ks;
 
+    constexpr int NOWHERE = 0x7fffffff; // past the end of either buffer
     lm_u32x4 rk[C::LOADS], rv[C::LOADS];
-    auto load = [&](lm_u32x4 (&r)[C::LOADS], const __amdgpu_buffer_rsrc_t rs, int d, int t) {
-        const int key0 = t * WA_KT, slot0 = key0 % p.cap;
+    int k_off[C::LOADS], v_off[C::LOADS]; // this lane's pieces of a tile whose first row is row 0
 #pragma unroll
-        for (int i = 0; i < C::LOADS; i++) {
-            const int x = i * 64 + lane, row = x / C::G, c = x % C::G, key = key0 + row;
-            int slot = slot0 + row;
-            if (slot >= p.cap) slot -= p.cap; // (a cache that wraps has more rows than a tile)
-            const int off = key >= lo_key && key <= last_pos && c * 8 < d ? (slot * d + c * 8) * 2 : 0x7fffffff;
-            r[i] = __builtin_bit_cast(lm_u32x4, __builtin_amdgcn_raw_buffer_load_b128(rs, off, 0, 0));
+    for (int i = 0; i < C::LOADS; i++) {
+        const int x = i * 64 + lane, row = x / C::G, c = x % C::G;
+        k_off[i] = c * 8 < p.dimp ? (row * p.dimp + c * 8) * 2 : NOWHERE;
+        v_off[i] = c * 8 < p.vdimp ? (row * p.vdimp + c * 8) * 2 : NOWHERE;
+    }
+    auto load = [&](lm_u32x4 (&r)[C::LOADS], const __amdgpu_buffer_rsrc_t rs, const int (&offs)[C::LOADS], int d, int t) {
+        const int key0 = __builtin_amdgcn_readfirstlane(t * WA_KT), slot0 = key0 % p.cap, row_bytes = d * 2;
+        if (key0 >= lo_key && key0 + WA_KT - 1 <= last_pos && slot0 + WA_KT <= p.cap) { // the whole tile, in one piece
+#pragma unroll
+            for (int i = 0; i < C::LOADS; i++) r[i] = __builtin_bit_cast(lm_u32x4, __builtin_amdgcn_raw_buffer_load_b128(rs, offs[i], slot0 * row_bytes, 0));
+        } else {
+#pragma unroll
+            for (int i = 0; i < C::LOADS; i++) {
+                const int row = (i * 64 + lane) / C::G, key = key0 + row;
+                int off = (offs[i] == NOWHERE ? 0 : offs[i]) + slot0 * row_bytes;
+                if (slot0 + row >= p.cap) off -= p.cap * row_bytes; // (a cache that wraps has more rows than a tile)
+                if (offs[i] == NOWHERE || key < lo_key || key > last_pos) off = NOWHERE;
+                r[i] = __builtin_bit_cast(lm_u32x4, __builtin_amdgcn_raw_buffer_load_b128(rs, off, 0, 0));
+            }
         }
     };
     auto store = [&](const lm_u32x4 (&r)[C::LOADS], bf16_t *dst, int stride) {
@@ -88,7 +102,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         }
     };
     int t = t_begin + wave;
-    if (C::AHEAD && t < t_end) load(rk, kr, p.dimp, t);
+    if (C::AHEAD && t < t_end) load(rk, kr, k_off, p.dimp, t);
     bf16x8_t qf[C::KSTEPS]; // the MFMA "B" operand: Q[row0 + col][16 s + 8 hf .. + 7]
     {
         const bf16_t *q = reinterpret_cast<const bf16_t *>(p.q) + size_t(min(row0 + col, p.n - 1)) * p.ldq + h * p.dimp;
@@ -96,10 +110,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         for (int s = 0; s < C::KSTEPS; s++) {
             lm_u32x4 v = {0, 0, 0, 0};
             if (16 * s + 8 * hf < p.dimp) v = *reinterpret_cast<const lm_u32x4 *>(q + 16 * s + 8 * hf);
+            if (p.scale < 0.0f) v ^= 0x80008000u; // scores are kept unscaled and the scale enters as its magnitude: the sign goes here
             qf[s] = __builtin_bit_cast(bf16x8_t, v);
         }
     }
-    if (C::AHEAD && t < t_end) load(rv, vr, p.vdimp, t);
+    if (C::AHEAD && t < t_end) load(rv, vr, v_off, p.vdimp, t);
     int voff[C::DT]; // where this lane points the transposing loads: key 4 hf + (lane % 16) / 4, columns 32 dt + 16 ((lane / 16) % 2) + 4 (lane % 4)
 #pragma unroll
     for (int dt = 0; dt < C::DT; dt++) voff[dt] = (4 * hf + ((lane & 15) >> 2)) * C::VS + 32 * dt + 16 * ((lane >> 4) & 1) + 4 * (lane & 3);
@@ -110,16 +125,16 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
 #pragma unroll
         for (int v = 0; v < 16; v++) o[dt][v] = 0.0f;
     constexpr float LOG2E = 1.4426950408889634f;
-    const float c2 = p.scale * LOG2E;
-    float m_run = -INFINITY, l_run = 0.0f; // in base-2 units; l_run: this lane's half of the row's sum
+    const float c2 = fmaxf(fabsf(p.scale) * LOG2E, 1e-37f); // > 0: the maximum of the scaled scores is the scaled maximum, -inf stays -inf
+    float m_run = -INFINITY, l_run = 0.0f; // m_run: scaled, in base-2 units; l_run: this lane's half of the row's sum
 
     for (; t < t_end; t += WA_WAVES) {
         const int key0 = t * WA_KT;
-        if (!C::AHEAD) load(rk, kr, p.dimp, t);
+        if (!C::AHEAD) load(rk, kr, k_off, p.dimp, t);
         asm volatile("" ::: "memory"); // the V tile of the round before has been read: the K tile takes its place
         store(rk, Ks, C::KS);
-        if (C::AHEAD && t + WA_WAVES < t_end) load(rk, kr, p.dimp, t + WA_WAVES);
-        if (!C::AHEAD) load(rv, vr, p.vdimp, t);
+        if (C::AHEAD && t + WA_WAVES < t_end) load(rk, kr, k_off, p.dimp, t + WA_WAVES);
+        if (!C::AHEAD) load(rv, vr, v_off, p.vdimp, t);
         float16_t s[2];
 #pragma unroll
         for (int kt = 0; kt < 2; kt++) {
@@ -133,12 +148,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         // s[kt][v]: key key0 + 32 kt + 8 (v / 4) + 4 hf + v % 4 against this lane's query
         float mx = -INFINITY;
         if (key0 + WA_KT - 1 > first_pos || (p.window && key0 < last_pos - p.window + 1)) { // some row does not see the whole tile
+            const int age0 = pos - key0 - 4 * hf; // how far back this lane's first key is
+            const unsigned ages = p.window ? (unsigned)p.window : 0x7fffffffu;
 #pragma unroll
             for (int kt = 0; kt < 2; kt++)
 #pragma unroll
-                for (int v = 0; v < 16; v++) {
-                    const int key = key0 + 32 * kt + 8 * (v >> 2) + 4 * hf + (v & 3);
-                    const float x = key > pos || (p.window && pos - key >= p.window) ? -INFINITY : s[kt][v] * c2;
+                for (int v = 0; v < 16; v++) { // (a key ahead of the query wraps to a large age)
+                    const float x = (unsigned)(age0 - (32 * kt + 8 * (v >> 2) + (v & 3))) < ages ? s[kt][v] : -INFINITY;
                     s[kt][v] = x;
                     mx = fmaxf(mx, x);
                 }
@@ -146,44 +162,46 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
 #pragma unroll
             for (int kt = 0; kt < 2; kt++)
 #pragma unroll
-                for (int v = 0; v < 16; v++) {
-                    s[kt][v] *= c2;
-                    mx = fmaxf(mx, s[kt][v]);
-                }
+                for (int v = 0; v < 16; v++) mx = fmaxf(mx, s[kt][v]);
         }
         mx = fmaxf(mx, __shfl_xor(mx, 32));
-        const float m_new = fmaxf(m_run, mx), m_use = m_new == -INFINITY ? 0.0f : m_new;
+        const float m_new = fmaxf(m_run, mx * c2), m_use = m_new == -INFINITY ? 0.0f : m_new;
         const float alpha = __builtin_amdgcn_exp2f(m_run - m_use);
+        const bool rescale = __any(m_new != m_run);
         m_run = m_new;
         float psum = 0.0f;
 #pragma unroll
         for (int kt = 0; kt < 2; kt++)
 #pragma unroll
             for (int v = 0; v < 16; v++) {
-                const float e = __builtin_amdgcn_exp2f(s[kt][v] - m_use);
+                const float e = __builtin_amdgcn_exp2f(__builtin_fmaf(s[kt][v], c2, -m_use));
                 s[kt][v] = e;
                 psum += e;
             }
         l_run = l_run * alpha + psum;
+        if (rescale)
 #pragma unroll
-        for (int dt = 0; dt < C::DT; dt++)
+            for (int dt = 0; dt < C::DT; dt++)
 #pragma unroll
-            for (int v = 0; v < 16; v++) o[dt][v] *= alpha;
+                for (int v = 0; v < 16; v++) o[dt][v] *= alpha;
         asm volatile("" ::: "memory"); // the K tile has been read (LDS serves a wavefront in order): V takes its place
         store(rv, Vs, C::VS);
-        if (C::AHEAD && t + WA_WAVES < t_end) load(rv, vr, p.vdimp, t + WA_WAVES);
+        if (C::AHEAD && t + WA_WAVES < t_end) load(rv, vr, v_off, p.vdimp, t + WA_WAVES);
         // contraction step (kt, sp) uses the keys a lane holds in s[kt][8 sp .. 8 sp + 7]: key0 + 32 kt + 16 sp + {4 hf + 0..3, 8 + 4 hf + 0..3}
 #pragma unroll
         for (int kt = 0; kt < 2; kt++)
 #pragma unroll
             for (int sp = 0; sp < 2; sp++) {
-                bf16x8_t hi, lo;
+                lm_u32x4 hi_bits, lo_bits; // two at a time: a packed conversion, its two halves back as f32, the remainders
 #pragma unroll
-                for (int e = 0; e < 8; e++) {
-                    const float w = s[kt][8 * sp + e];
-                    hi[e] = (bf16_t)w;
-                    lo[e] = (bf16_t)(w - (float)hi[e]);
+                for (int e = 0; e < 4; e++) {
+                    const float2_t w = {s[kt][8 * sp + 2 * e], s[kt][8 * sp + 2 * e + 1]};
+                    hi_bits[e] = __builtin_bit_cast(unsigned, __builtin_convertvector(w, bf16x2_t));
+                    const unsigned pair = hi_bits[e];
+                    const float2_t rest = {w[0] - __builtin_bit_cast(float, pair << 16), w[1] - __builtin_bit_cast(float, pair & 0xffff0000u)};
+                    lo_bits[e] = __builtin_bit_cast(unsigned, __builtin_convertvector(rest, bf16x2_t));
                 }
+                const bf16x8_t hi = __builtin_bit_cast(bf16x8_t, hi_bits), lo = __builtin_bit_cast(bf16x8_t, lo_bits);
 #pragma unroll
                 for (int dt = 0; dt < C::DT; dt++) {
                     const bf16_t *vp = Vs + voff[dt] + (32 * kt + 16 * sp) * C::VS;
@@ -195,6 +213,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
             }
     }
 
+    // this thread's gate values for the merged result, requested before the merge
+    const int q = tid & 31, row = row0 + q, d0 = (tid >> 5) * 8;
+    const bf16_t *gate = p.gate ? reinterpret_cast<const bf16_t *>(p.gate) + size_t(min(row, p.n - 1)) * p.ldq + h * p.vdimp : nullptr;
+    bf16x8_t gz = {};
+    if (gate && d0 < p.vdimp) gz = *reinterpret_cast<const bf16x8_t *>(gate + d0);
     // merge the wavefronts' results; the sink is one more term of the denominator
     const float l_wave = l_run + __shfl_xor(l_run, 32);
     float *so = reinterpret_cast<float *>(wa_lds), *sm = reinterpret_cast<float *>(reinterpret_cast<char *>(wa_lds) + C::ML_OFFSET), *sl = sm + WA_WAVES * WA_Q;
@@ -216,7 +239,6 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
             *reinterpret_cast<float4 *>(so + (wave * WA_Q + col) * C::SD + 32 * dt + 8 * j + 4 * hf) = r;
         }
     __syncthreads();
-    const int q = tid & 31, row = row0 + q;
     if (row >= p.n) return;
     float l_all = p.sink ? __builtin_amdgcn_exp2f(sink - m_all) : 0.0f;
 #pragma unroll
@@ -225,16 +247,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         if (mw != -INFINITY) l_all += __builtin_amdgcn_exp2f(mw - m_all) * sl[w * WA_Q + q];
     }
     const float inv = 1.0f / l_all;
-    const bf16_t *gate = p.gate ? reinterpret_cast<const bf16_t *>(p.gate) + size_t(row) * p.ldq + h * p.vdimp : nullptr;
     bf16_t *out = reinterpret_cast<bf16_t *>(p.out) + size_t(row) * p.ldo + h * p.vdimp;
-    for (int d = (tid >> 5) * 8; d < p.vdimp; d += 64) {
+    for (int d = d0; d < p.vdimp; d += 64) {
         float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int w = 0; w < WA_WAVES; w++)
 #pragma unroll
             for (int e = 0; e < 8; e++) acc[e] += so[(w * WA_Q + q) * C::SD + d + e];
-        bf16x8_t gz = {}, r;
-        if (gate) gz = *reinterpret_cast<const bf16x8_t *>(gate + d);
+        bf16x8_t r;
+        if (gate && d != d0) gz = *reinterpret_cast<const bf16x8_t *>(gate + d);
 #pragma unroll
         for (int e = 0; e < 8; e++) r[e] = (bf16_t)(acc[e] * inv * (gate ? lm_sigmoid((float)gz[e]) : 1.0f));
         *reinterpret_cast<bf16x8_t *>(out + d) = r;

@@ -12,6 +12,7 @@
 #include "router.hpp"
 
 #include <algorithm>
+#include <type_traits>
 
 namespace {
 
@@ -50,9 +51,10 @@ struct RowDots {
 // Row of gate/up column pair i (half 0: gate, 1: up) in the interleaved weights
 __device__ __forceinline__ int pair_row(int i, int half) { return (i >> 5) * 64 + half * 32 + (i & 31); }
 
-template <class T, int U>
+// NV: 16-byte pieces of x, gamma and beta a thread holds (rows of up to 1024 NV elements, a multiple of 4); 0: any row, from memory
+template <class T, int U, int NV>
 __global__ __launch_bounds__(256) void decode_proj_kernel(DecodeProj p) {
-    extern __shared__ __attribute__((aligned(16))) char s_raw[]; // h: T [dp], then x: float [width]
+    extern __shared__ __attribute__((aligned(16))) char s_raw[]; // h: T [dp], then (NV = 0) x: float [width]
     T *s_h = reinterpret_cast<T *>(s_raw);
     float *s_x = reinterpret_cast<float *>(s_raw + size_t(p.dp) * sizeof(T));
     __shared__ float s_red[16];
@@ -76,30 +78,75 @@ __global__ __launch_bounds__(256) void decode_proj_kernel(DecodeProj p) {
             rows[j] = W + size_t(row) * p.dp; // (segments are padded to whole groups)
         }
     };
+    // The norm's inputs are requested first, then the first weights: loads return in order, so the weights stream in while the
+    // norm is computed.
+    const T *er = p.token ? reinterpret_cast<const T *>(p.embed) + size_t(p.token[0]) * p.dp : nullptr;
+    float4_t xv[NV ? NV : 1], gv[NV ? NV : 1], bv[NV ? NV : 1];
+    if (NV) {
+#pragma unroll
+        for (int k = 0; k < NV; k++) {
+            const int i = (k * 256 + tid) * 4, j = i < p.width ? i : 0;
+            if (er) {
+#pragma unroll
+                for (int e = 0; e < 4; e++) xv[k][e] = (float)er[j + e];
+            } else xv[k] = *reinterpret_cast<const float4_t *>(p.x + j);
+            gv[k] = *reinterpret_cast<const float4_t *>(p.gamma + j);
+            bv[k] = *reinterpret_cast<const float4_t *>(p.beta + j);
+        }
+    }
     RowDots<T, RG, U> dots;
-    if (g_begin < g_end) { // the first weights stream in while the norm is computed
+    if (g_begin < g_end) {
         locate(g_begin);
         dots.request(rows, 0, pieces, lane);
     }
-    const T *er = p.token ? reinterpret_cast<const T *>(p.embed) + size_t(p.token[0]) * p.dp : nullptr;
-    float s = 0.0f;
-    for (int i = tid; i < p.width; i += 256) {
-        const float v = er ? (float)er[i] * p.embed_scale : p.x[i];
-        if (er && blockIdx.x == 0) p.x[i] = v;
-        s_x[i] = v;
-        s += v;
-    }
-    const float mean = block_sum(s, s_red) / (float)p.width;
-    float m2 = 0.0f;
-    for (int i = tid; i < p.width; i += 256) {
-        const float d = s_x[i] - mean;
-        m2 = fmaf(d, d, m2);
-    }
-    const float rstd = 1.0f / sqrtf(block_sum(m2, s_red) / (float)p.width + p.eps);
-    for (int i = tid; i < p.dp; i += 256) {
-        const T v = i < p.width ? (T)((s_x[i] - mean) * rstd * p.gamma[i] + p.beta[i]) : (T)0.0f;
-        s_h[i] = v;
-        if (p.h && blockIdx.x == 0) reinterpret_cast<T *>(p.h)[i] = v;
+    float s = 0.0f, m2 = 0.0f;
+    if (NV) {
+#pragma unroll
+        for (int k = 0; k < NV; k++) {
+            const int i = (k * 256 + tid) * 4;
+            if (er) xv[k] *= p.embed_scale;
+            if (i >= p.width) xv[k] = float4_t{0, 0, 0, 0};
+            else if (er && blockIdx.x == 0) *reinterpret_cast<float4_t *>(p.x + i) = xv[k];
+            s += (xv[k][0] + xv[k][1]) + (xv[k][2] + xv[k][3]);
+        }
+        const float mean = block_sum(s, s_red) / (float)p.width;
+#pragma unroll
+        for (int k = 0; k < NV; k++)
+            if ((k * 256 + tid) * 4 < p.width) {
+                xv[k] -= mean;
+#pragma unroll
+                for (int e = 0; e < 4; e++) m2 = fmaf(xv[k][e], xv[k][e], m2);
+            }
+        const float rstd = 1.0f / sqrtf(block_sum(m2, s_red) / (float)p.width + p.eps);
+#pragma unroll
+        for (int k = 0; k < NV; k++) {
+            const int i = (k * 256 + tid) * 4;
+            if (i >= p.dp) continue;
+            typedef T vec4 __attribute__((ext_vector_type(4)));
+            vec4 v;
+#pragma unroll
+            for (int e = 0; e < 4; e++) v[e] = i < p.width ? (T)(xv[k][e] * rstd * gv[k][e] + bv[k][e]) : (T)0.0f;
+            *reinterpret_cast<vec4 *>(s_h + i) = v;
+            if (p.h && blockIdx.x == 0) *reinterpret_cast<vec4 *>(reinterpret_cast<T *>(p.h) + i) = v;
+        }
+    } else {
+        for (int i = tid; i < p.width; i += 256) {
+            const float v = er ? (float)er[i] * p.embed_scale : p.x[i];
+            if (er && blockIdx.x == 0) p.x[i] = v;
+            s_x[i] = v;
+            s += v;
+        }
+        const float mean = block_sum(s, s_red) / (float)p.width;
+        for (int i = tid; i < p.width; i += 256) {
+            const float d = s_x[i] - mean;
+            m2 = fmaf(d, d, m2);
+        }
+        const float rstd = 1.0f / sqrtf(block_sum(m2, s_red) / (float)p.width + p.eps);
+        for (int i = tid; i < p.dp; i += 256) {
+            const T v = i < p.width ? (T)((s_x[i] - mean) * rstd * p.gamma[i] + p.beta[i]) : (T)0.0f;
+            s_h[i] = v;
+            if (p.h && blockIdx.x == 0) reinterpret_cast<T *>(p.h)[i] = v;
+        }
     }
     lds_barrier();
     for (int g = g_begin; g < g_end; g++) {
@@ -130,7 +177,7 @@ __global__ __launch_bounds__(256) void decode_proj_kernel(DecodeProj p) {
 
 constexpr int MIX_HEADS = 8;       // query heads one workgroup serves
 constexpr int MIX_KEYS = 1024;     // keys of one split at most
-constexpr int MIX_TARGET = 64;     // keys of one split at least
+constexpr int MIX_TARGET = 32;     // keys of one split at least
 __host__ __device__ __forceinline__ int mix_head_blocks(int per_group) { return (per_group + MIX_HEADS - 1) / MIX_HEADS; }
 
 __device__ __forceinline__ int next_pow2(int v) { return v <= 1 ? 1 : 1 << (32 - __builtin_clz(v - 1)); }
@@ -305,16 +352,27 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
     }
     __syncthreads();
     if (!*s_last) return;
-    // All of a head's splits: the weight of each (a lane per split) to LDS, then the sums with several loads in flight.
+    // Every head's splits: this thread's elements of the first splits and all (m, l) are requested together; the weight of each
+    // split (a lane per split) goes through LDS.
+    constexpr int AT_ONCE = 16;
+    const size_t pitch = size_t(MIX_HEADS) * stride; // floats between splits
     float *s_w = lds; // [nh][S], over what the phases before have used
+    float v[AT_ONCE];
+    {
+        const int i = min(tid, nh * p.vdimp - 1);
+        const float *ph = part + size_t(i / p.vdimp) * stride + i % p.vdimp;
+#pragma unroll
+        for (int u = 0; u < AT_ONCE; u++) v[u] = ld_f<true>(ph + min(u, S - 1) * pitch);
+    }
     for (int h = wave; h < nh; h += 4) {
         const float *ph = part + size_t(h) * stride + p.vdimp, sink = p.sink ? p.sink[h0 + h] : -INFINITY;
-        float m = sink, l = 0.0f;
-        for (int s = lane; s < S; s += 64) m = fmaxf(m, ld_f<true>(ph + size_t(s) * MIX_HEADS * stride));
+        const float m0 = lane < S ? ld_f<true>(ph + lane * pitch) : -INFINITY, l0 = lane < S ? ld_f<true>(ph + lane * pitch + 1) : 0.0f;
+        float m = fmaxf(sink, m0), l = 0.0f;
+        for (int s = lane + 64; s < S; s += 64) m = fmaxf(m, ld_f<true>(ph + s * pitch));
         m = wave_max(m);
-        for (int s = lane; s < S; s += 64) {
-            const float w = expf(ld_f<true>(ph + size_t(s) * MIX_HEADS * stride) - m); // (an empty split: m = -inf, weight 0)
-            l = fmaf(ld_f<true>(ph + size_t(s) * MIX_HEADS * stride + 1), w, l);
+        for (int s = lane; s < S; s += 64) { // (an empty split: m = -inf, weight 0)
+            const float w = expf((s == lane ? m0 : ld_f<true>(ph + s * pitch)) - m);
+            l = fmaf(s == lane ? l0 : ld_f<true>(ph + s * pitch + 1), w, l);
             s_w[h * S + s] = w;
         }
         l = wave_sum(l) + (p.sink ? expf(sink - m) : 0.0f);
@@ -324,12 +382,11 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
     for (int i = tid; i < nh * p.vdimp; i += 256) {
         const int h = i / p.vdimp, d = i % p.vdimp;
         const float *ph = part + size_t(h) * stride + d;
-        constexpr int AT_ONCE = 8;
         float o = 0.0f;
         for (int s0 = 0; s0 < S; s0 += AT_ONCE) {
-            float v[AT_ONCE];
+            if (s0 || i != tid)
 #pragma unroll
-            for (int u = 0; u < AT_ONCE; u++) v[u] = ld_f<true>(ph + size_t(min(s0 + u, S - 1)) * MIX_HEADS * stride);
+                for (int u = 0; u < AT_ONCE; u++) v[u] = ld_f<true>(ph + min(s0 + u, S - 1) * pitch);
 #pragma unroll
             for (int u = 0; u < AT_ONCE; u++)
                 if (s0 + u < S) o = fmaf(v[u], s_w[h * S + s0 + u], o);
@@ -461,11 +518,16 @@ template <class T, int NH> int mix_launch(moon_ctx *ctx, const DecodeMix &p, int
 template <class T> int proj_launch(moon_ctx *ctx, const DecodeProj &p) {
     const int cus = ctx->cu_count > 0 ? ctx->cu_count : 256;
     const int groups = (p.n16_used + 3) / 4 + (p.n32_used + 3) / 4 + (p.ff + 1) / 2;
-    const dim3 grid((unsigned)std::max(1, std::min(4 * cus, (groups + 3) / 4)));
-    const size_t lds = size_t(p.dp) * sizeof(T) + size_t(p.width) * sizeof(float);
-    const int ch = (p.dp / Piece<T>::N + 63) / 64;
-    auto kern = ch == 1 ? decode_proj_kernel<T, 1> : ch == 2 ? decode_proj_kernel<T, 2> : ch == 3 ? decode_proj_kernel<T, 3> : decode_proj_kernel<T, 4>;
+    const dim3 grid((unsigned)std::max(1, std::min(2 * cus, (groups + 3) / 4)));
+    const int ch = (p.dp / Piece<T>::N + 63) / 64, nv = p.width % 4 || p.dp > 4096 || (reinterpret_cast<uintptr_t>(p.x) & 15) ? 0 : (p.dp + 1023) / 1024;
+    const size_t lds = size_t(p.dp) * sizeof(T) + (nv ? 0 : size_t(p.width) * sizeof(float));
     if (lds > 60 * 1024) return moon_fail(ctx, MOON_EINVAL_DIM, "decode: width %d too large", p.width);
+    auto pick = [&](auto u) {
+        constexpr int U = decltype(u)::value;
+        return nv == 0 ? decode_proj_kernel<T, U, 0> : nv == 1 ? decode_proj_kernel<T, U, 1> : nv == 2 ? decode_proj_kernel<T, U, 2> : decode_proj_kernel<T, U, 4>;
+    };
+    auto kern = ch == 1 ? pick(std::integral_constant<int, 1>{}) : ch == 2 ? pick(std::integral_constant<int, 2>{}) : ch == 3 ? pick(std::integral_constant<int, 3>{})
+                                                                                                                          : pick(std::integral_constant<int, 4>{});
     hipLaunchKernelGGL(kern, grid, dim3(256), lds, ctx->stream, p);
     MOON_HIP(ctx, hipGetLastError());
     return MOON_OK;
@@ -493,13 +555,13 @@ int launch_decode_out(moon_ctx *ctx, int dtype, const DecodeOut &p) {
 size_t decode_mix_counters(size_t heads, size_t kv_heads) { return kv_heads * mix_head_blocks((int)(heads / kv_heads)); }
 size_t decode_mix_partial_floats(moon_ctx *ctx, size_t heads, size_t kv_heads, size_t vdimp, size_t max_keys) {
     const size_t cus = ctx->cu_count > 0 ? ctx->cu_count : 256, wgs = decode_mix_counters(heads, kv_heads);
-    return std::max(std::max(wgs, 2 * cus), wgs * ((max_keys + MIX_KEYS - 1) / MIX_KEYS)) * MIX_HEADS * (vdimp + 2);
+    return std::max(std::max(wgs, cus), wgs * ((max_keys + MIX_KEYS - 1) / MIX_KEYS)) * MIX_HEADS * (vdimp + 2);
 }
 
 int launch_decode_mix(moon_ctx *ctx, int dtype, const DecodeMix &p) {
     const int cus = ctx->cu_count > 0 ? ctx->cu_count : 256, per = p.H / p.G, wgs = p.G * mix_head_blocks(per);
     const int n_keys = (int)(p.window ? std::min(p.pos + 1, (size_t)p.window) : p.pos + 1);
-    int S = std::min((n_keys + MIX_TARGET - 1) / MIX_TARGET, std::max(1, 2 * cus / wgs));
+    int S = std::min((n_keys + MIX_TARGET - 1) / MIX_TARGET, std::max(1, cus / wgs));
     S = std::max(S, (n_keys + MIX_KEYS - 1) / MIX_KEYS);
     if (size_t(wgs) * S * MIX_HEADS * (p.vdimp + 2) > p.partial_floats) return moon_fail(ctx, MOON_ESEQ_TOO_LONG, "decode attention: %d keys", n_keys);
     const int keys_max = (n_keys + S - 1) / S;

@@ -162,7 +162,15 @@ __global__ __launch_bounds__(1024) void group_kernel(RouteArgs p) {
     const int per = (total + 15) / 16, lo = min(wave * per, total), hi = min(lo + per, total); // a wavefront's run of pairs
     for (int e = tid; e < 16 * p.E; e += 1024) per_wave[e] = 0;
     __syncthreads();
-    for (int i = lo + lane; i < hi; i += 64) atomicAdd(&per_wave[wave * p.E + p.ids[i]], 1);
+    constexpr int AHEAD = 8; // ids requested together
+    for (int base = lo; base < hi; base += 64 * AHEAD) {
+        int e[AHEAD];
+#pragma unroll
+        for (int u = 0; u < AHEAD; u++) e[u] = base + u * 64 + lane < hi ? p.ids[base + u * 64 + lane] : -1;
+#pragma unroll
+        for (int u = 0; u < AHEAD; u++)
+            if (e[u] >= 0) atomicAdd(&per_wave[wave * p.E + e[u]], 1);
+    }
     __syncthreads();
     for (int e = tid; e < p.E; e += 1024) { // rows of expert e
         int c = 0;
@@ -193,9 +201,10 @@ __global__ __launch_bounds__(1024) void group_kernel(RouteArgs p) {
             p.tile_row[t] = start[e] + (t - tiles[e]) * p.rows_per_tile;
             p.tile_end[t] = start[e + 1];
         }
+    int next = lo + lane < hi ? p.ids[lo + lane] : -1;
     for (int base = lo; base < hi; base += 64) { // 64 pairs at a time, in order
-        const int i = base + lane;
-        const int e = i < hi ? p.ids[i] : -1;
+        const int i = base + lane, e = next;
+        next = i + 64 < hi ? p.ids[i + 64] : -1;
         unsigned long long match = ~0ull; // the lanes with this lane's expert
         for (int bit = 1; bit < 2 * p.E; bit <<= 1) { // (lanes past the end count as expert E)
             const unsigned long long ones = __ballot(((e < 0 ? p.E : e) & bit) != 0);
