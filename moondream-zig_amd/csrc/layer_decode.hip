@@ -178,6 +178,7 @@ __global__ __launch_bounds__(256) void decode_proj_kernel(DecodeProj p) {
 constexpr int MIX_HEADS = 8;       // query heads one workgroup serves
 constexpr int MIX_KEYS = 1024;     // keys of one split at most
 constexpr int MIX_TARGET = 32;     // keys of one split at least
+constexpr int MIX_SPLITS = 16;     // splits at most, unless MIX_KEYS asks for more: what the merge requests at once
 __host__ __device__ __forceinline__ int mix_head_blocks(int per_group) { return (per_group + MIX_HEADS - 1) / MIX_HEADS; }
 
 __device__ __forceinline__ int next_pow2(int v) { return v <= 1 ? 1 : 1 << (32 - __builtin_clz(v - 1)); }
@@ -185,6 +186,32 @@ __device__ __forceinline__ int next_pow2(int v) { return v <= 1 ? 1 : 1 << (32 -
 // LDS of an attention workgroup, in floats: q [NH][dimp], new k [dimp], new v [vdimp], scores [NH][keys], reduction [4][NH][vdimp], misc
 __host__ __device__ __forceinline__ size_t mix_lds_floats(int nh, int dimp, int vdimp, int keys) {
     return size_t(nh) * dimp + dimp + vdimp + size_t(nh) * keys + size_t(4) * nh * vdimp + 4 * nh + 8; // (launch_decode_mix: at least nh * S before the misc)
+}
+
+// Sums of N values over the lanes that differ in the bits of OFF and below down to `stop` (a power of two, the same in every lane).
+// At every step a lane hands one half of its values to its partner and keeps the other, so N / 2 + N / 4 + .. exchanges do; done(i, sum)
+// is called for the values that end up in this lane (by several lanes where there are fewer values than lanes).
+template <int N, int OFF, class Done>
+__device__ __forceinline__ void fold_lanes(float (&v)[N], int lane, int stop, int base, Done done) {
+    if (OFF < stop) {
+#pragma unroll
+        for (int i = 0; i < N; i++) done(base + i, v[i]);
+        return;
+    }
+    const bool upper = lane & OFF;
+    if constexpr (N > 1) {
+        float half[N / 2];
+#pragma unroll
+        for (int i = 0; i < N / 2; i++) half[i] = (upper ? v[i + N / 2] : v[i]) + __shfl_xor(upper ? v[i] : v[i + N / 2], OFF);
+        if constexpr (OFF > 1) fold_lanes<N / 2, OFF / 2>(half, lane, stop, base + (upper ? N / 2 : 0), done);
+        else
+#pragma unroll
+            for (int i = 0; i < N / 2; i++) done(base + (upper ? N / 2 : 0) + i, half[i]);
+    } else {
+        v[0] += __shfl_xor(v[0], OFF);
+        if constexpr (OFF > 1) fold_lanes<1, OFF / 2>(v, lane, stop, base, done);
+        else done(base, v[0]);
+    }
 }
 
 // Attention of one token: kv head g, query heads h0 .. h0 + nh - 1, split `split` of S.
@@ -323,13 +350,14 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
             }
             for (int key = j0 + (PF * 4 + wave) * vpw + vsub; key < j1; key += 4 * vpw) value_step(key, key == pos ? pv[0] : v_piece(key, c));
         }
+        float flat[NH * PE];
 #pragma unroll
         for (int h = 0; h < NH; h++)
 #pragma unroll
-            for (int e = 0; e < PE; e++) {
-                for (int off = 32; off >= lpv; off >>= 1) acc[h][e] += __shfl_xor(acc[h][e], off);
-                if (vsub == 0 && c < vp && h < nh) s_r[(wave * NH + h) * p.vdimp + c * PE + e] = acc[h][e];
-            }
+            for (int e = 0; e < PE; e++) flat[h * PE + e] = acc[h][e];
+        fold_lanes<NH * PE, 32>(flat, lane, lpv, 0, [&](int i, float v) {
+            if (c < vp && i / PE < nh) s_r[(wave * NH + i / PE) * p.vdimp + c * PE + i % PE] = v;
+        });
     }
     lds_barrier();
     // This split's sums and (m, l) per head to memory; the workgroup that counts in last adds the splits up.
@@ -354,7 +382,7 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
     if (!*s_last) return;
     // Every head's splits: this thread's elements of the first splits and all (m, l) are requested together; the weight of each
     // split (a lane per split) goes through LDS.
-    constexpr int AT_ONCE = 16;
+    constexpr int AT_ONCE = MIX_SPLITS;
     const size_t pitch = size_t(MIX_HEADS) * stride; // floats between splits
     float *s_w = lds; // [nh][S], over what the phases before have used
     float v[AT_ONCE];
@@ -419,20 +447,32 @@ __device__ __forceinline__ void mix_experts(const DecodeMix &p, int wg, int n_wg
     share(p.top * per_expert, n_wgs * 4, wg * 4 + wave, g_begin, g_end);
     RowDots<T, RG, U> dots;
     const T *rows[RG];
-    for (int g = g_begin; g < g_end; g++) {
+    auto locate = [&](int g) {
         const int k = g / per_expert, i = 2 * (g % per_expert);
         const T *W = reinterpret_cast<const T *>(p.wgu) + size_t(s_ids[k]) * 2 * p.ffp * p.dp;
 #pragma unroll
         for (int j = 0; j < RG; j++) rows[j] = W + size_t(pair_row(i + (j >> 1), j & 1)) * p.dp;
+    };
+    if (g_begin < g_end) {
+        locate(g_begin);
+        dots.request(rows, 0, pieces, lane);
+    }
+    for (int g = g_begin; g < g_end; g++) {
         float acc[RG] = {0.0f, 0.0f, 0.0f, 0.0f};
-        for (int p0 = 0; p0 < pieces; p0 += 64 * U) {
-            dots.request(rows, p0, pieces, lane);
+        for (int p0 = 0;;) {
             dots.add(s_h, p0, pieces, lane, acc);
+            p0 += 64 * U;
+            if (p0 >= pieces) break;
+            dots.request(rows, p0, pieces, lane);
+        }
+        if (g + 1 < g_end) {
+            locate(g + 1);
+            dots.request(rows, 0, pieces, lane);
         }
 #pragma unroll
         for (int j = 0; j < RG; j++) acc[j] = wave_sum(acc[j]);
         if (lane == 0) {
-            T *o = reinterpret_cast<T *>(p.act) + size_t(k) * p.ffp + i;
+            T *o = reinterpret_cast<T *>(p.act) + size_t(g / per_expert) * p.ffp + 2 * (g % per_expert);
             o[0] = (T)(lm_silu(acc[0]) * acc[1]);
             o[1] = (T)(lm_silu(acc[2]) * acc[3]);
         }
@@ -442,13 +482,10 @@ __device__ __forceinline__ void mix_experts(const DecodeMix &p, int wg, int n_wg
 template <class T, int NH, int U>
 __global__ __launch_bounds__(256) void decode_mix_kernel(DecodeMix p, int S, int keys_max, int n_attn, int n_expert) {
     extern __shared__ __attribute__((aligned(16))) char s_mix[];
-    // expert workgroups first: they have the most to read
-    if ((int)blockIdx.x < n_expert) {
-        mix_experts<T, U>(p, blockIdx.x, n_expert, s_mix);
-        return;
-    }
-    const int i = blockIdx.x - n_expert, n_hb = mix_head_blocks(p.H / p.G);
-    mix_attention<T, NH>(p, i / S / n_hb, i / S % n_hb, i % S, S, keys_max, reinterpret_cast<float *>(s_mix));
+    // attention first: it is a chain of dependent steps, the experts' part is one long stream
+    const int i = blockIdx.x, n_hb = mix_head_blocks(p.H / p.G);
+    if (i < n_attn) mix_attention<T, NH>(p, i / S / n_hb, i / S % n_hb, i % S, S, keys_max, reinterpret_cast<float *>(s_mix));
+    else mix_experts<T, U>(p, i - n_attn, n_expert, s_mix);
 }
 
 // x[n] += sum over the pieces of row n of W2 against a, and of the chosen experts' rows against their activations.  A workgroup
@@ -561,13 +598,13 @@ size_t decode_mix_partial_floats(moon_ctx *ctx, size_t heads, size_t kv_heads, s
 int launch_decode_mix(moon_ctx *ctx, int dtype, const DecodeMix &p) {
     const int cus = ctx->cu_count > 0 ? ctx->cu_count : 256, per = p.H / p.G, wgs = p.G * mix_head_blocks(per);
     const int n_keys = (int)(p.window ? std::min(p.pos + 1, (size_t)p.window) : p.pos + 1);
-    int S = std::min((n_keys + MIX_TARGET - 1) / MIX_TARGET, std::max(1, cus / wgs));
+    int S = std::min(std::min((n_keys + MIX_TARGET - 1) / MIX_TARGET, MIX_SPLITS), std::max(1, cus / wgs));
     S = std::max(S, (n_keys + MIX_KEYS - 1) / MIX_KEYS);
     if (size_t(wgs) * S * MIX_HEADS * (p.vdimp + 2) > p.partial_floats) return moon_fail(ctx, MOON_ESEQ_TOO_LONG, "decode attention: %d keys", n_keys);
     const int keys_max = (n_keys + S - 1) / S;
     if (p.E && (p.top < 1 || p.top > p.E || p.E > ROUTER_MAX_EXPERTS)) return moon_fail(ctx, MOON_EINVAL_DIM, "router: %d of %d experts", p.top, p.E);
     const int groups = p.E ? p.top * ((p.ff + 1) / 2) : 0;
-    const int n_expert = std::min((groups + 3) / 4, std::max(cus, 2 * cus - wgs * S));
+    const int n_expert = std::min((groups + 3) / 4, std::max(cus, 2 * cus - wgs * S)); // (together two workgroups per CU: more measured slower)
     const int nh = std::min(per, MIX_HEADS), NH = nh <= 1 ? 1 : nh <= 2 ? 2 : nh <= 4 ? 4 : 8;
     const size_t el = dtype == MOON_DTYPE_BF16 ? sizeof(bf16_t) : sizeof(float);
     const size_t lds = std::max(mix_lds_floats(NH, p.dimp, p.vdimp, keys_max) * sizeof(float),
