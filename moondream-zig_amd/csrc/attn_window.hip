@@ -26,9 +26,11 @@ typedef float float2_t __attribute__((ext_vector_type(2)));
 
 template <int P> struct WaCfg { // P: head sizes up to P (a multiple of 32), rows zero padded to it
     static constexpr int KSTEPS = P / 16, DT = P / 32, G = P / 8;
-    static constexpr int KS = P + 8; // row strides in elements: 128-bit reads of consecutive K rows and the transposing reads of
-    static constexpr int VS = P == 32 ? 32 : P <= 96 ? 96 : P + 32; // 4 consecutive V rows (16 dwords apart mod 64) are conflict free
-    static constexpr int WAVE_ELEMS = WA_KT * (KS > VS ? KS : VS);  // K is only read before the scores, V only after: they share the area
+    static constexpr int KS = P + 8; // K row stride: 128-bit reads of consecutive rows are conflict free
+    // V rows are unpadded.  The transposing reads take 16 dwords of each of 4 consecutive rows: rows of 16 or 48 dwords lie apart
+    // mod 64 by themselves, in the others granule c of row r sits at c ^ SWZ * (r % 4).
+    static constexpr int VS = P, SWZ = P == 64 ? 2 : P >= 128 ? 4 : 0;
+    static constexpr int WAVE_ELEMS = WA_KT * KS; // K is only read before the scores, V only after: they share the area
     static constexpr int LOADS = G;  // 16-byte pieces per lane and operand tile
     static constexpr bool AHEAD = P <= 128; // the next tile's pieces wait in registers (above, there are too many)
     static constexpr int SD = P + 4; // merge: O as [wave][q][SD] floats, (m, l) [wave][q] behind them
@@ -79,7 +81,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         v_off[i] = c * 8 < p.vdimp ? (row * p.vdimp + c * 8) * 2 : NOWHERE;
     }
     auto load = [&](lm_u32x4 (&r)[C::LOADS], const __amdgpu_buffer_rsrc_t rs, const int (&offs)[C::LOADS], int d, int t) {
-        const int key0 = __builtin_amdgcn_readfirstlane(t * WA_KT), slot0 = key0 % p.cap, row_bytes = d * 2;
+        const int key0 = __builtin_amdgcn_readfirstlane(t * WA_KT), slot0 = key0 < p.cap ? key0 : key0 % p.cap, row_bytes = d * 2;
         if (key0 >= lo_key && key0 + WA_KT - 1 <= last_pos && slot0 + WA_KT <= p.cap) { // the whole tile, in one piece
 #pragma unroll
             for (int i = 0; i < C::LOADS; i++) r[i] = __builtin_bit_cast(lm_u32x4, __builtin_amdgcn_raw_buffer_load_b128(rs, offs[i], slot0 * row_bytes, 0));
@@ -94,11 +96,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
             }
         }
     };
-    auto store = [&](const lm_u32x4 (&r)[C::LOADS], bf16_t *dst, int stride) {
+    auto store = [&](const lm_u32x4 (&r)[C::LOADS], bf16_t *dst, int stride, int swz) {
 #pragma unroll
         for (int i = 0; i < C::LOADS; i++) {
-            const int x = i * 64 + lane;
-            *reinterpret_cast<lm_u32x4 *>(dst + x / C::G * stride + x % C::G * 8) = r[i];
+            const int x = i * 64 + lane, row = x / C::G;
+            *reinterpret_cast<lm_u32x4 *>(dst + row * stride + (x % C::G ^ swz * (row & 3)) * 8) = r[i];
         }
     };
     int t = t_begin + wave;
@@ -117,7 +119,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
     if (C::AHEAD && t < t_end) load(rv, vr, v_off, p.vdimp, t);
     int voff[C::DT]; // where this lane points the transposing loads: key 4 hf + (lane % 16) / 4, columns 32 dt + 16 ((lane / 16) % 2) + 4 (lane % 4)
 #pragma unroll
-    for (int dt = 0; dt < C::DT; dt++) voff[dt] = (4 * hf + ((lane & 15) >> 2)) * C::VS + 32 * dt + 16 * ((lane >> 4) & 1) + 4 * (lane & 3);
+    for (int dt = 0; dt < C::DT; dt++) {
+        const int rq = (lane & 15) >> 2, d = 32 * dt + 16 * ((lane >> 4) & 1) + 4 * (lane & 3);
+        voff[dt] = (4 * hf + rq) * C::VS + ((d >> 3 ^ C::SWZ * rq) << 3 | (d & 7));
+    }
 
     float16_t o[C::DT];
 #pragma unroll
@@ -126,13 +131,14 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         for (int v = 0; v < 16; v++) o[dt][v] = 0.0f;
     constexpr float LOG2E = 1.4426950408889634f;
     const float c2 = fmaxf(fabsf(p.scale) * LOG2E, 1e-37f); // > 0: the maximum of the scaled scores is the scaled maximum, -inf stays -inf
+    const float sink = p.sink ? p.sink[h] * LOG2E : -INFINITY;
     float m_run = -INFINITY, l_run = 0.0f; // m_run: scaled, in base-2 units; l_run: this lane's half of the row's sum
 
     for (; t < t_end; t += WA_WAVES) {
         const int key0 = t * WA_KT;
         if (!C::AHEAD) load(rk, kr, k_off, p.dimp, t);
         asm volatile("" ::: "memory"); // the V tile of the round before has been read: the K tile takes its place
-        store(rk, Ks, C::KS);
+        store(rk, Ks, C::KS, 0);
         if (C::AHEAD && t + WA_WAVES < t_end) load(rk, kr, k_off, p.dimp, t + WA_WAVES);
         if (!C::AHEAD) load(rv, vr, v_off, p.vdimp, t);
         float16_t s[2];
@@ -185,7 +191,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
 #pragma unroll
                 for (int v = 0; v < 16; v++) o[dt][v] *= alpha;
         asm volatile("" ::: "memory"); // the K tile has been read (LDS serves a wavefront in order): V takes its place
-        store(rv, Vs, C::VS);
+        store(rv, Vs, C::VS, C::SWZ);
         if (C::AHEAD && t + WA_WAVES < t_end) load(rv, vr, v_off, p.vdimp, t + WA_WAVES);
         // contraction step (kt, sp) uses the keys a lane holds in s[kt][8 sp .. 8 sp + 7]: key0 + 32 kt + 16 sp + {4 hf + 0..3, 8 + 4 hf + 0..3}
 #pragma unroll
@@ -226,7 +232,6 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         sl[wave * WA_Q + col] = l_wave;
     }
     __syncthreads(); // every wavefront is done with its staging area
-    const float sink = p.sink ? p.sink[h] * LOG2E : -INFINITY;
     float m_all = sink;
 #pragma unroll
     for (int w = 0; w < WA_WAVES; w++) m_all = fmaxf(m_all, sm[w * WA_Q + col]);
