@@ -1,5 +1,6 @@
-// Causal attention of several query rows over a KV cache, with a sliding window, grouped key/value heads, a sink in the
-// softmax denominator and an output gate; each of them is an argument.  The cache of a layer is [G][cap][head size]; the keys of
+// Causal attention of several query rows over a KV cache, with a sliding window, pooled blocks before it, grouped key/value heads, a
+// sink in the softmax denominator, a factor per head on the scale, outputs that turn back by their position's angles (where the values
+// were turned by theirs) and an output gate; each of them is an argument.  The cache of a layer is [G][cap][head size]; the keys of
 // position p lie in row p % cap, so a windowed layer needs no more rows than its window and one call's rows together.
 //
 // bf16 runs on the matrix cores, arranged like the kernel of attn_prefill.hip: a 256-thread workgroup owns 32 query rows of one
@@ -18,6 +19,9 @@
 #include <atomic>
 
 namespace {
+
+// Blocks that lie wholly before the window of position pos: block b ends at b pool + pool - 1 <= pos - window
+__device__ __forceinline__ int blocks_seen(int pos, int window, int pool) { return max(0, pos - window + 1) / pool; }
 
 constexpr int WA_KT = 64, WA_Q = 32, WA_WAVES = 4; // keys per tile, query rows and wavefronts per workgroup
 typedef short wa_short4_t __attribute__((ext_vector_type(4)));
@@ -43,7 +47,8 @@ __device__ __forceinline__ wa_short4_t wa_read_tr(const bf16_t *p) {
     return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) wa_short4_t *)(p));
 }
 
-template <int P>
+// POOL: the tiles of the blocks' keys come first, in the same softmax
+template <int P, bool POOL>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2 : 1))) void window_attn_kernel(WindowAttn p) {
     using C = WaCfg<P>;
     extern __shared__ __attribute__((aligned(16))) bf16_t wa_lds[];
@@ -64,11 +69,16 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
     const int g = h / (p.H / p.G), row0 = qb * WA_Q;
     const int first_pos = p.pos0 + row0, last_pos = p.pos0 + min(row0 + WA_Q, p.n) - 1, pos = first_pos + col; // pos: this lane's query
     const int lo_key = p.window ? max(0, first_pos - p.window + 1) : 0;
-    const int t_begin = lo_key / WA_KT, t_end = last_pos / WA_KT + 1; // tiles start at multiples of 64 positions
+    // tiles start at multiples of 64 positions; POOL: tile numbers below t_window stand for blocks (of the first one, from 0 on)
+    const int seen = POOL ? blocks_seen(last_pos, p.window, p.pool) : 0, t_blocks = (seen + WA_KT - 1) / WA_KT;
+    const int t_begin = POOL ? lo_key / WA_KT - t_blocks : lo_key / WA_KT, t_end = last_pos / WA_KT + 1;
+    const int t_window = POOL ? lo_key / WA_KT : 0;
     // the head's cache rows as buffers: a 32-bit offset per piece, and what must not be read is an offset past the end (zeros)
     const int k_bytes = p.cap * p.dimp * 2, v_bytes = p.cap * p.vdimp * 2;
     const __amdgpu_buffer_rsrc_t kr = __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t *>(reinterpret_cast<const bf16_t *>(p.ck) + size_t(g) * p.cap * p.dimp), 0, k_bytes, 0x00020000);
     const __amdgpu_buffer_rsrc_t vr = __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t *>(reinterpret_cast<const bf16_t *>(p.cv) + size_t(g) * p.cap * p.vdimp), 0, v_bytes, 0x00020000);
+    const __amdgpu_buffer_rsrc_t pkr = __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t *>(reinterpret_cast<const bf16_t *>(p.pk) + size_t(g) * p.blocks * p.dimp), 0, POOL ? p.blocks * p.dimp * 2 : 0, 0x00020000);
+    const __amdgpu_buffer_rsrc_t pvr = __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t *>(reinterpret_cast<const bf16_t *>(p.pv) + size_t(g) * p.blocks * p.vdimp), 0, POOL ? p.blocks * p.vdimp * 2 : 0, 0x00020000);
     bf16_t *Ks = wa_lds + wave * C::WAVE_ELEMS, *Vs = Ks;
 
     constexpr int NOWHERE = 0x7fffffff; // past the end of either buffer
@@ -80,7 +90,16 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         k_off[i] = c * 8 < p.dimp ? (row * p.dimp + c * 8) * 2 : NOWHERE;
         v_off[i] = c * 8 < p.vdimp ? (row * p.vdimp + c * 8) * 2 : NOWHERE;
     }
-    auto load = [&](lm_u32x4 (&r)[C::LOADS], const __amdgpu_buffer_rsrc_t rs, const int (&offs)[C::LOADS], int d, int t) {
+    auto load = [&](lm_u32x4 (&r)[C::LOADS], const __amdgpu_buffer_rsrc_t rs, const __amdgpu_buffer_rsrc_t blocks, const int (&offs)[C::LOADS], int d, int t) {
+        if (POOL && t < t_window) {
+            const int b0 = __builtin_amdgcn_readfirstlane((t - t_begin) * WA_KT);
+#pragma unroll
+            for (int i = 0; i < C::LOADS; i++) {
+                const int off = offs[i] == NOWHERE || b0 + (i * 64 + lane) / C::G >= seen ? NOWHERE : offs[i] + b0 * d * 2;
+                r[i] = __builtin_bit_cast(lm_u32x4, __builtin_amdgcn_raw_buffer_load_b128(blocks, off, 0, 0));
+            }
+            return;
+        }
         const int key0 = __builtin_amdgcn_readfirstlane(t * WA_KT), slot0 = key0 < p.cap ? key0 : key0 % p.cap, row_bytes = d * 2;
         if (key0 >= lo_key && key0 + WA_KT - 1 <= last_pos && slot0 + WA_KT <= p.cap) { // the whole tile, in one piece
 #pragma unroll
@@ -104,7 +123,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         }
     };
     int t = t_begin + wave;
-    if (C::AHEAD && t < t_end) load(rk, kr, k_off, p.dimp, t);
+    if (C::AHEAD && t < t_end) load(rk, kr, pkr, k_off, p.dimp, t);
+    const float scale = p.temp ? p.scale * p.temp[h] : p.scale;
     bf16x8_t qf[C::KSTEPS]; // the MFMA "B" operand: Q[row0 + col][16 s + 8 hf .. + 7]
     {
         const bf16_t *q = reinterpret_cast<const bf16_t *>(p.q) + size_t(min(row0 + col, p.n - 1)) * p.ldq + h * p.dimp;
@@ -112,11 +132,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         for (int s = 0; s < C::KSTEPS; s++) {
             lm_u32x4 v = {0, 0, 0, 0};
             if (16 * s + 8 * hf < p.dimp) v = *reinterpret_cast<const lm_u32x4 *>(q + 16 * s + 8 * hf);
-            if (p.scale < 0.0f) v ^= 0x80008000u; // scores are kept unscaled and the scale enters as its magnitude: the sign goes here
+            if (scale < 0.0f) v ^= 0x80008000u; // scores are kept unscaled and the scale enters as its magnitude: the sign goes here
             qf[s] = __builtin_bit_cast(bf16x8_t, v);
         }
     }
-    if (C::AHEAD && t < t_end) load(rv, vr, v_off, p.vdimp, t);
+    if (C::AHEAD && t < t_end) load(rv, vr, pvr, v_off, p.vdimp, t);
     int voff[C::DT]; // where this lane points the transposing loads: key 4 hf + (lane % 16) / 4, columns 32 dt + 16 ((lane / 16) % 2) + 4 (lane % 4)
 #pragma unroll
     for (int dt = 0; dt < C::DT; dt++) {
@@ -130,17 +150,17 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
 #pragma unroll
         for (int v = 0; v < 16; v++) o[dt][v] = 0.0f;
     constexpr float LOG2E = 1.4426950408889634f;
-    const float c2 = fmaxf(fabsf(p.scale) * LOG2E, 1e-37f); // > 0: the maximum of the scaled scores is the scaled maximum, -inf stays -inf
+    const float c2 = fmaxf(fabsf(scale) * LOG2E, 1e-37f); // > 0: the maximum of the scaled scores is the scaled maximum, -inf stays -inf
     const float sink = p.sink ? p.sink[h] * LOG2E : -INFINITY;
     float m_run = -INFINITY, l_run = 0.0f; // m_run: scaled, in base-2 units; l_run: this lane's half of the row's sum
 
     for (; t < t_end; t += WA_WAVES) {
         const int key0 = t * WA_KT;
-        if (!C::AHEAD) load(rk, kr, k_off, p.dimp, t);
+        if (!C::AHEAD) load(rk, kr, pkr, k_off, p.dimp, t);
         asm volatile("" ::: "memory"); // the V tile of the round before has been read: the K tile takes its place
         store(rk, Ks, C::KS, 0);
-        if (C::AHEAD && t + WA_WAVES < t_end) load(rk, kr, k_off, p.dimp, t + WA_WAVES);
-        if (!C::AHEAD) load(rv, vr, v_off, p.vdimp, t);
+        if (C::AHEAD && t + WA_WAVES < t_end) load(rk, kr, pkr, k_off, p.dimp, t + WA_WAVES);
+        if (!C::AHEAD) load(rv, vr, pvr, v_off, p.vdimp, t);
         float16_t s[2];
 #pragma unroll
         for (int kt = 0; kt < 2; kt++) {
@@ -153,7 +173,17 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         }
         // s[kt][v]: key key0 + 32 kt + 8 (v / 4) + 4 hf + v % 4 against this lane's query
         float mx = -INFINITY;
-        if (key0 + WA_KT - 1 > first_pos || (p.window && key0 < last_pos - p.window + 1)) { // some row does not see the whole tile
+        if (POOL && t < t_window) {
+            const int mine = blocks_seen(pos, p.window, p.pool) - (t - t_begin) * WA_KT - 4 * hf;
+#pragma unroll
+            for (int kt = 0; kt < 2; kt++)
+#pragma unroll
+                for (int v = 0; v < 16; v++) {
+                    const float x = 32 * kt + 8 * (v >> 2) + (v & 3) < mine ? s[kt][v] : -INFINITY;
+                    s[kt][v] = x;
+                    mx = fmaxf(mx, x);
+                }
+        } else if (key0 + WA_KT - 1 > first_pos || (p.window && key0 < last_pos - p.window + 1)) { // some row does not see the whole tile
             const int age0 = pos - key0 - 4 * hf; // how far back this lane's first key is
             const unsigned ages = p.window ? (unsigned)p.window : 0x7fffffffu;
 #pragma unroll
@@ -192,7 +222,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
                 for (int v = 0; v < 16; v++) o[dt][v] *= alpha;
         asm volatile("" ::: "memory"); // the K tile has been read (LDS serves a wavefront in order): V takes its place
         store(rv, Vs, C::VS, C::SWZ);
-        if (C::AHEAD && t + WA_WAVES < t_end) load(rv, vr, v_off, p.vdimp, t + WA_WAVES);
+        if (C::AHEAD && t + WA_WAVES < t_end) load(rv, vr, pvr, v_off, p.vdimp, t + WA_WAVES);
         // contraction step (kt, sp) uses the keys a lane holds in s[kt][8 sp .. 8 sp + 7]: key0 + 32 kt + 16 sp + {4 hf + 0..3, 8 + 4 hf + 0..3}
 #pragma unroll
         for (int kt = 0; kt < 2; kt++)
@@ -259,10 +289,27 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(P <= 64 ? 2
         for (int w = 0; w < WA_WAVES; w++)
 #pragma unroll
             for (int e = 0; e < 8; e++) acc[e] += so[(w * WA_Q + q) * C::SD + d + e];
+#pragma unroll
+        for (int e = 0; e < 8; e++) acc[e] *= inv;
+        if (p.rotv) { // each element with the other one of its pair
+            const int half = p.vdim / 2;
+#pragma unroll
+            for (int e = 0; e < 8; e++)
+                if (d + e < 2 * half) {
+                    const bool second = d + e >= half;
+                    const int m = second ? d + e - half : d + e, other = second ? m : m + half;
+                    const float2 cs = p.rotv[size_t(p.pos0 + row) * half + m];
+                    float z = 0.0f;
+#pragma unroll
+                    for (int w = 0; w < WA_WAVES; w++) z += so[(w * WA_Q + q) * C::SD + other];
+                    z *= inv;
+                    acc[e] = second ? acc[e] * cs.x - z * cs.y : acc[e] * cs.x + z * cs.y;
+                }
+        }
         bf16x8_t r;
         if (gate && d != d0) gz = *reinterpret_cast<const bf16x8_t *>(gate + d);
 #pragma unroll
-        for (int e = 0; e < 8; e++) r[e] = (bf16_t)(acc[e] * inv * (gate ? lm_sigmoid((float)gz[e]) : 1.0f));
+        for (int e = 0; e < 8; e++) r[e] = (bf16_t)(acc[e] * (gate ? lm_sigmoid((float)gz[e]) : 1.0f));
         *reinterpret_cast<bf16x8_t *>(out + d) = r;
     }
 }
@@ -279,20 +326,24 @@ __global__ __launch_bounds__(256) void window_attn_rows_kernel(WindowAttn p) {
     const T *ck = reinterpret_cast<const T *>(p.ck) + size_t(g) * p.cap * p.dimp, *cv = reinterpret_cast<const T *>(p.cv) + size_t(g) * p.cap * p.vdimp;
     for (int d = lane; d < p.dimp; d += 64) s_q[wave][d] = (float)q[d];
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    const float scale = p.temp ? p.scale * p.temp[h] : p.scale;
+    const int seen = p.pool ? blocks_seen(pos, p.window, p.pool) : 0; // the blocks come first, then the tokens from lo on
+    const T *pk = reinterpret_cast<const T *>(p.pk) + size_t(g) * p.blocks * p.dimp, *pv = reinterpret_cast<const T *>(p.pv) + size_t(g) * p.blocks * p.vdimp;
     float m = p.sink ? p.sink[h] : -INFINITY, l = p.sink ? 1.0f : 0.0f;
     float o[ROW_MAX_D / 64];
 #pragma unroll
     for (int i = 0; i < ROW_MAX_D / 64; i++) o[i] = 0.0f;
-    for (int k0 = lo; k0 <= pos; k0 += 64) {
-        const int key = k0 + lane, n_keys = min(64, pos - k0 + 1);
+    const int total = seen + pos - lo + 1;
+    for (int k0 = 0; k0 < total; k0 += 64) {
+        const int key = k0 + lane, n_keys = min(64, total - k0);
         float s = -INFINITY;
-        if (key <= pos) {
-            const T *kr = ck + size_t(key % p.cap) * p.dimp;
+        if (key < total) {
+            const T *kr = key < seen ? pk + size_t(key) * p.dimp : ck + size_t((key - seen + lo) % p.cap) * p.dimp;
             s = 0.0f;
             for (int d = 0; d < p.dimp; d++) s = fmaf(s_q[wave][d], (float)kr[d], s);
-            s *= p.scale;
+            s *= scale;
         }
-        const float m_new = fmaxf(m, wave_max(s)), alpha = expf(m - m_new), w = key <= pos ? expf(s - m_new) : 0.0f;
+        const float m_new = fmaxf(m, wave_max(s)), alpha = expf(m - m_new), w = key < total ? expf(s - m_new) : 0.0f;
         l = l * alpha + wave_sum(w);
         m = m_new;
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -304,33 +355,44 @@ __global__ __launch_bounds__(256) void window_attn_rows_kernel(WindowAttn p) {
             if (64 * i >= p.vdimp) continue;
             float acc = o[i] * alpha;
             if (d < p.vdimp)
-                for (int j = 0; j < n_keys; j++) acc = fmaf(s_w[wave][j], (float)cv[size_t((k0 + j) % p.cap) * p.vdimp + d], acc);
+                for (int j = 0; j < n_keys; j++) {
+                    const int at = k0 + j;
+                    acc = fmaf(s_w[wave][j], (float)(at < seen ? pv + size_t(at) * p.vdimp : cv + size_t((at - seen + lo) % p.cap) * p.vdimp)[d], acc);
+                }
             o[i] = acc;
         }
     }
 #pragma unroll
-    for (int i = 0; i < ROW_MAX_D / 64; i++) {
-        const int d = 64 * i + lane;
-        if (d >= p.vdimp) continue;
-        float r = o[i] / l;
+    for (int i = 0; i < ROW_MAX_D / 64; i++)
+        if (64 * i + lane < p.vdimp) s_q[wave][64 * i + lane] = o[i] / l; // (the query is not needed any more)
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    const int half = p.rotv ? p.vdim / 2 : 0;
+    for (int d = lane; d < p.vdimp; d += 64) {
+        float r = s_q[wave][d];
+        if (d < 2 * half) {
+            const int m = d < half ? d : d - half;
+            const float2 cs = p.rotv[size_t(pos) * half + m];
+            r = d < half ? r * cs.x + s_q[wave][d + half] * cs.y : r * cs.x - s_q[wave][m] * cs.y;
+        }
         if (p.gate) r *= lm_sigmoid((float)reinterpret_cast<const T *>(p.gate)[size_t(row) * p.ldq + h * p.vdimp + d]);
         reinterpret_cast<T *>(p.out)[size_t(row) * p.ldo + h * p.vdimp + d] = (T)r;
     }
 }
 
-template <int P> int launch_mfma(moon_ctx *ctx, const WindowAttn &p) {
+template <int P, bool POOL> int launch_mfma_as(moon_ctx *ctx, const WindowAttn &p) {
     using C = WaCfg<P>;
     static std::atomic<bool> attr_set[64]; // the opt-in to this much dynamic LDS is per device (and per instantiation)
     const int dev = ctx->device >= 0 && ctx->device < 64 ? ctx->device : -1;
     if (dev < 0 || !attr_set[dev].load()) {
-        MOON_HIP(ctx, hipFuncSetAttribute(reinterpret_cast<const void *>(window_attn_kernel<P>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)C::LDS_BYTES));
+        MOON_HIP(ctx, hipFuncSetAttribute(reinterpret_cast<const void *>(window_attn_kernel<P, POOL>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)C::LDS_BYTES));
         if (dev >= 0) attr_set[dev].store(true);
     }
-    hipLaunchKernelGGL(window_attn_kernel<P>, dim3((unsigned)((p.n + WA_Q - 1) / WA_Q * p.H)), dim3(256), C::LDS_BYTES, ctx->stream, p);
+    hipLaunchKernelGGL((window_attn_kernel<P, POOL>), dim3((unsigned)((p.n + WA_Q - 1) / WA_Q * p.H)), dim3(256), C::LDS_BYTES, ctx->stream, p);
     MOON_HIP(ctx, hipGetLastError());
     MOON_NOTE_KERNEL(ctx, "window_attn_kernel<%d>", P);
     return MOON_OK;
 }
+template <int P> int launch_mfma(moon_ctx *ctx, const WindowAttn &p) { return p.pool ? launch_mfma_as<P, true>(ctx, p) : launch_mfma_as<P, false>(ctx, p); }
 
 } // namespace
 
@@ -340,8 +402,10 @@ int launch_window_attention(moon_ctx *ctx, int dtype, const WindowAttn &p) {
         return moon_fail(ctx, MOON_EINVAL_DIM, "window attention: %d heads over %d, head sizes %d and %d", p.H, p.G, p.dimp, p.vdimp);
     if ((p.window ? p.window - 1 + p.n : p.pos0 + p.n) > p.cap && p.pos0 + p.n > p.cap)
         return moon_fail(ctx, MOON_EINVAL_DIM, "window attention: %d rows behind a window of %d do not fit %d cache rows", p.n, p.window, p.cap);
+    if (p.pool && (!p.window || (p.pos0 + p.n - p.window) / p.pool > p.blocks)) // (no block is seen before it is whole)
+        return moon_fail(ctx, MOON_EINVAL_DIM, "window attention: blocks of %d before a window of %d, %d of them kept", p.pool, p.window, p.blocks);
     const int big = std::max(p.dimp, p.vdimp);
-    if (dtype == MOON_DTYPE_BF16 && big <= 256 && size_t(p.cap) * big * 2 < (size_t(1) << 30)) { // (32-bit offsets within a head's rows)
+    if (dtype == MOON_DTYPE_BF16 && big <= 256 && size_t(std::max(p.cap, p.blocks)) * big * 2 < (size_t(1) << 30)) { // (32-bit offsets within a head's rows)
         if (big <= 32) return launch_mfma<32>(ctx, p);
         if (big <= 64) return launch_mfma<64>(ctx, p);
         if (big <= 96) return launch_mfma<96>(ctx, p);

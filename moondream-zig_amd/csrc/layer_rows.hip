@@ -1,5 +1,5 @@
-// Row-wise kernels of the layer-list decoders: embedding, residual sum and LayerNorm; q/k norm, value mixing and the cache
-// update of a prompt's rows; the router and the grouping of rows by expert.
+// Row-wise kernels of the layer-list decoders: embedding, residual sum and norm; q/k norm, rotation, value mixing and the cache
+// update of a prompt's rows; the means of blocks of cache rows; the router and the grouping of rows by expert.
 #include "layer_list.hpp"
 #include "lm_types.hpp"
 #include "norm.hpp"
@@ -29,17 +29,18 @@ template <class T> struct RowVec<T, 4> {
     }
 };
 
-// W: elements a thread takes at a time (4 where the width allows)
-template <class T, int W>
+// W: elements a thread takes at a time (4 where the width allows).  JOIN: the first splits are two outputs that are normed first.
+template <class T, int W, bool JOIN>
 __global__ __launch_bounds__(256) void row_finish_kernel(RowFinish p) {
-    extern __shared__ __attribute__((aligned(16))) float s_row[]; // [width]
+    extern __shared__ __attribute__((aligned(16))) float s_row[]; // [width], JOIN: and the two outputs
     __shared__ float sm[16];
     const int r = blockIdx.x, tid = threadIdx.x;
     float *xr = p.x + size_t(p.rows ? p.rows[r] : (uint32_t)r) * p.width;
     const T *er = p.embed ? reinterpret_cast<const T *>(p.embed) + size_t(p.ids[r]) * p.dp : nullptr;
     const T *eo = reinterpret_cast<const T *>(p.expert_out);
     const bool changes = er || p.splits || p.top;
-    float s = 0.0f;
+    float s = 0.0f, ss_l = 0.0f, ss_r = 0.0f;
+    float *s_l = s_row + p.width, *s_r = s_l + p.width; // (JOIN only)
     for (int i = tid * W; i < p.width; i += 256 * W) {
         float v[W], d[W] = {};
         if (er) {
@@ -48,8 +49,27 @@ __global__ __launch_bounds__(256) void row_finish_kernel(RowFinish p) {
             for (int e = 0; e < W; e++) v[e] *= p.embed_scale;
         } else {
             RowVec<float, W>::load(xr + i, v);
+            if (JOIN) {
+                float l[W] = {}, r2[W] = {};
 #pragma unroll 4
-            for (int k = 0; k < p.splits; k++) {
+                for (int k = 0; k < p.splits_l + p.splits_r; k++) {
+                    float t[W];
+                    RowVec<float, W>::load(p.partial + (size_t(k) * p.n + r) * p.dp + i, t);
+#pragma unroll
+                    for (int e = 0; e < W; e++)
+                        if (k < p.splits_l) l[e] += t[e];
+                        else r2[e] += t[e];
+                }
+#pragma unroll
+                for (int e = 0; e < W; e++) {
+                    ss_l = fmaf(l[e], l[e], ss_l);
+                    ss_r = fmaf(r2[e], r2[e], ss_r);
+                }
+                RowVec<float, W>::store(s_l + i, l);
+                RowVec<float, W>::store(s_r + i, r2);
+            }
+#pragma unroll 4
+            for (int k = JOIN ? p.splits_l + p.splits_r : 0; k < p.splits; k++) {
                 float t[W];
                 RowVec<float, W>::load(p.partial + (size_t(k) * p.n + r) * p.dp + i, t);
 #pragma unroll
@@ -66,13 +86,32 @@ __global__ __launch_bounds__(256) void row_finish_kernel(RowFinish p) {
 #pragma unroll
             for (int e = 0; e < W; e++) v[e] += d[e];
         }
-        if (changes) RowVec<float, W>::store(xr + i, v);
+        if (changes && !JOIN) RowVec<float, W>::store(xr + i, v);
         RowVec<float, W>::store(s_row + i, v);
 #pragma unroll
         for (int e = 0; e < W; e++) s += v[e];
     }
+    if (JOIN) { // (each thread reads back what it wrote)
+        const float f_l = 0.5f / sqrtf(block_sum(ss_l, sm) / (float)p.width + p.eps), f_r = 0.5f / sqrtf(block_sum(ss_r, sm) / (float)p.width + p.eps);
+        s = 0.0f;
+        for (int i = tid * W; i < p.width; i += 256 * W) {
+            float v[W], l[W], r2[W], wl[W], wr[W];
+            RowVec<float, W>::load(s_row + i, v);
+            RowVec<float, W>::load(s_l + i, l);
+            RowVec<float, W>::load(s_r + i, r2);
+            RowVec<float, W>::load(p.out_l + i, wl);
+            RowVec<float, W>::load(p.out_r + i, wr);
+#pragma unroll
+            for (int e = 0; e < W; e++) {
+                v[e] += l[e] * f_l * wl[e] + r2[e] * f_r * wr[e];
+                s += v[e];
+            }
+            RowVec<float, W>::store(xr + i, v);
+            RowVec<float, W>::store(s_row + i, v);
+        }
+    }
     if (!p.h) return;
-    const float mean = block_sum(s, sm) / (float)p.width;
+    const float mean = p.beta ? block_sum(s, sm) / (float)p.width : 0.0f; // (an RMS norm takes no mean off)
     float m2 = 0.0f;
     for (int i = tid * W; i < p.width; i += 256 * W) // (each thread reads back what it wrote)
 #pragma unroll
@@ -86,9 +125,9 @@ __global__ __launch_bounds__(256) void row_finish_kernel(RowFinish p) {
         float v[W] = {}, ga[W], be[W];
         if (i < p.width) {
             RowVec<float, W>::load(p.gamma + i, ga);
-            RowVec<float, W>::load(p.beta + i, be);
+            if (p.beta) RowVec<float, W>::load(p.beta + i, be);
 #pragma unroll
-            for (int e = 0; e < W; e++) v[e] = (s_row[i + e] - mean) * rstd * ga[e] + be[e];
+            for (int e = 0; e < W; e++) v[e] = (s_row[i + e] - mean) * rstd * ga[e] + (p.beta ? be[e] : 0.0f);
         }
         RowVec<T, W>::store(h + i, v);
     }
@@ -143,6 +182,92 @@ __global__ __launch_bounds__(256) void prep_qkv_kernel(PrepArgs p, int lph) {
             *reinterpret_cast<lm_u32x4 *>(dst + c * PE) = o;
         }
     }
+}
+
+// One workgroup per row: q and k as a whole through their norms, heads of q, k and v turned, k and v into the cache.
+template <class T>
+__global__ __launch_bounds__(256) void prep_whole_kernel(PrepWhole p) {
+    extern __shared__ __attribute__((aligned(16))) float s_qkv[]; // q, k, v
+    __shared__ float sm[16];
+    constexpr int PE = Piece<T>::N;
+    const int tid = threadIdx.x, r = blockIdx.x, pos = p.pos0 + r, slot = p.G ? pos % p.cap : 0;
+    const int nq = p.H * p.dimp, nk = p.G * p.dimp, nv = p.G * p.vdimp;
+    T *row = reinterpret_cast<T *>(p.c1) + size_t(r) * p.ld;
+    float ss_q = 0.0f, ss_k = 0.0f;
+    for (int i = tid * PE; i < nq + nk + nv; i += 256 * PE) {
+        float v[PE];
+        Piece<T>::unpack(*reinterpret_cast<const lm_u32x4 *>(row + (i < nq ? p.oq + i : i < nq + nk ? p.ok + i - nq : p.ov + i - nq - nk)), v);
+        float s = 0.0f;
+#pragma unroll
+        for (int e = 0; e < PE; e++) {
+            s = fmaf(v[e], v[e], s);
+            s_qkv[i + e] = v[e];
+        }
+        if (i < nq) ss_q += s;
+        else if (i < nq + nk) ss_k += s;
+    }
+    const float f_q = 1.0f / sqrtf(block_sum(ss_q, sm) / (float)(p.H * p.dim) + p.eps); // (its barriers also order the copy in LDS)
+    const float f_k = p.G ? 1.0f / sqrtf(block_sum(ss_k, sm) / (float)(p.G * p.dim) + p.eps) : 0.0f;
+    for (int i = tid * PE; i < nq + nk + nv; i += 256 * PE) {
+        const bool is_v = i >= nq + nk, is_q = i < nq;
+        const int at = is_q ? i : is_v ? i - nq - nk : i - nq, size = is_v ? p.vdimp : p.dimp, head = at / size, d0 = at % size;
+        const float *x = s_qkv + i - d0, *w = is_v ? nullptr : (is_q ? p.qn : p.kn) + at - d0; // this head's elements and weights
+        const float f = is_v ? 1.0f : is_q ? f_q : f_k;
+        const float2 *table = is_v ? p.rotv : p.rot;
+        const int half = !table ? 0 : (is_v ? p.vdim : p.rot_dims) / 2;
+        lm_u32x4 o;
+        T *t = reinterpret_cast<T *>(&o);
+#pragma unroll
+        for (int e = 0; e < PE; e++) {
+            const int d = d0 + e;
+            float y = w ? x[d] * f * w[d] : x[d];
+            if (d < 2 * half) {
+                const int m = d < half ? d : d - half, other = d < half ? d + half : m;
+                const float2 cs = table[size_t(pos) * half + m];
+                const float z = w ? x[other] * f * w[other] : x[other];
+                y = d < half ? y * cs.x - z * cs.y : y * cs.x + z * cs.y;
+            }
+            t[e] = (T)y;
+        }
+        T *dst = is_q ? row + p.oq + i : is_v ? reinterpret_cast<T *>(p.cv) + (size_t(head) * p.cap + slot) * p.vdimp + d0
+                                              : reinterpret_cast<T *>(p.ck) + (size_t(head) * p.cap + slot) * p.dimp + d0;
+        *reinterpret_cast<lm_u32x4 *>(dst) = o;
+    }
+}
+
+// 16 bytes of a block's row per thread
+template <class T>
+__global__ __launch_bounds__(256) void pool_kernel(PoolArgs p, int first, int tasks) {
+    constexpr int PE = Piece<T>::N;
+    const int i = blockIdx.x * 256 + threadIdx.x, pk = p.dimp / PE, per_head = pk + p.vdimp / PE;
+    if (i >= tasks) return;
+    const int piece = i % per_head, g = i / per_head % p.G, b = first + i / per_head / p.G;
+    const bool is_v = piece >= pk;
+    const int size = is_v ? p.vdimp : p.dimp, d = (is_v ? piece - pk : piece) * PE;
+    const T *src = reinterpret_cast<const T *>(is_v ? p.cv : p.ck) + size_t(g) * p.cap * size + d;
+    float acc[PE];
+#pragma unroll
+    for (int e = 0; e < PE; e++) acc[e] = 0.0f;
+#pragma unroll 4
+    for (int j = 0; j < p.pool; j++) {
+        float v[PE];
+        Piece<T>::unpack(*reinterpret_cast<const lm_u32x4 *>(src + size_t((b * p.pool + j) % p.cap) * size), v);
+#pragma unroll
+        for (int e = 0; e < PE; e++) acc[e] += v[e];
+    }
+    lm_u32x4 o;
+    T *t = reinterpret_cast<T *>(&o);
+#pragma unroll
+    for (int e = 0; e < PE; e++) t[e] = (T)(acc[e] / (float)p.pool);
+    *reinterpret_cast<lm_u32x4 *>(reinterpret_cast<T *>(is_v ? p.pv : p.pk) + (size_t(g) * p.blocks + b) * size + d) = o;
+}
+
+__global__ __launch_bounds__(256) void rotation_table_kernel(float2 *table, size_t n, int half, double base, double factor) {
+    const size_t i = size_t(blockIdx.x) * 256 + threadIdx.x;
+    if (i >= n) return;
+    double s, c;
+    sincos(double(i / half) * (pow(base, -double(i % half) / half) / factor), &s, &c);
+    table[i] = float2{(float)c, (float)s};
 }
 
 __global__ __launch_bounds__(256) void route_kernel(RouteArgs p) {
@@ -224,13 +349,54 @@ __global__ __launch_bounds__(1024) void group_kernel(RouteArgs p) {
 
 } // namespace
 
+template <class T> static int row_finish_launch(moon_ctx *ctx, const RowFinish &p) {
+    const bool join = p.out_l != nullptr;
+    const size_t lds = size_t(p.width) * sizeof(float) * (join ? 3 : 1);
+    if (lds > 156 * 1024) return moon_fail(ctx, MOON_EINVAL_DIM, "row kernel: width %d too large", p.width);
+    auto kern = join ? (p.width % 4 ? row_finish_kernel<T, 1, true> : row_finish_kernel<T, 4, true>)
+                     : (p.width % 4 ? row_finish_kernel<T, 1, false> : row_finish_kernel<T, 4, false>);
+    if (lds > 60 * 1024) MOON_HIP(ctx, hipFuncSetAttribute(reinterpret_cast<const void *>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    hipLaunchKernelGGL(kern, dim3(p.n), dim3(256), lds, ctx->stream, p);
+    MOON_HIP(ctx, hipGetLastError());
+    return MOON_OK;
+}
 int launch_row_finish(moon_ctx *ctx, int dtype, const RowFinish &p) {
     if (p.n <= 0) return MOON_OK;
-    const size_t lds = size_t(p.width) * sizeof(float);
-    if (lds > 60 * 1024) return moon_fail(ctx, MOON_EINVAL_DIM, "row kernel: width %d too large", p.width);
-    auto kern = dtype == MOON_DTYPE_BF16 ? (p.width % 4 ? row_finish_kernel<bf16_t, 1> : row_finish_kernel<bf16_t, 4>)
-                                         : (p.width % 4 ? row_finish_kernel<float, 1> : row_finish_kernel<float, 4>);
+    if (p.out_l && (p.splits_l < 1 || p.splits_r < 1 || p.splits_l + p.splits_r > p.splits || p.embed))
+        return moon_fail(ctx, MOON_EINVAL, "row kernel: %d and %d of %d splits are joined", p.splits_l, p.splits_r, p.splits);
+    return dtype == MOON_DTYPE_BF16 ? row_finish_launch<bf16_t>(ctx, p) : row_finish_launch<float>(ctx, p);
+}
+
+int launch_prep_whole(moon_ctx *ctx, int dtype, const PrepWhole &p) {
+    if (p.n <= 0) return MOON_OK;
+    if (p.G && p.n > p.cap) return moon_fail(ctx, MOON_EINVAL_DIM, "cache update: %d rows, %d slots", p.n, p.cap);
+    if (p.dimp % 8 || p.vdimp % 8 || p.rot_dims % 2 || p.rot_dims > p.dim || (p.rotv && p.vdim % 2))
+        return moon_fail(ctx, MOON_EINVAL_DIM, "cache update: head sizes %d and %d, %d dimensions turn", p.dim, p.vdim, p.rot_dims);
+    const size_t lds = (size_t(p.H + p.G) * p.dimp + size_t(p.G) * p.vdimp) * sizeof(float);
+    if (lds > 156 * 1024) return moon_fail(ctx, MOON_EINVAL_DIM, "cache update: %d heads too wide for one workgroup", p.H);
+    auto kern = dtype == MOON_DTYPE_BF16 ? prep_whole_kernel<bf16_t> : prep_whole_kernel<float>;
+    if (lds > 60 * 1024) MOON_HIP(ctx, hipFuncSetAttribute(reinterpret_cast<const void *>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
     hipLaunchKernelGGL(kern, dim3(p.n), dim3(256), lds, ctx->stream, p);
+    MOON_HIP(ctx, hipGetLastError());
+    return MOON_OK;
+}
+
+int launch_pool(moon_ctx *ctx, int dtype, const PoolArgs &p) {
+    const int first = p.pos0 / p.pool, blocks = (p.pos0 + p.n) / p.pool - first;
+    if (p.n <= 0 || blocks <= 0) return MOON_OK;
+    if (first + blocks > p.blocks || (p.pool - 1 + p.n > p.cap && p.pos0 + p.n > p.cap))
+        return moon_fail(ctx, MOON_EINVAL_DIM, "pooled blocks: %d of %d blocks, %d rows behind %d positions", first + blocks, p.blocks, p.n, p.pool);
+    const int tasks = blocks * p.G * (p.dimp + p.vdimp) / (dtype == MOON_DTYPE_BF16 ? Piece<bf16_t>::N : Piece<float>::N);
+    auto kern = dtype == MOON_DTYPE_BF16 ? pool_kernel<bf16_t> : pool_kernel<float>;
+    hipLaunchKernelGGL(kern, dim3((unsigned)(tasks + 255) / 256), dim3(256), 0, ctx->stream, p, first, tasks);
+    MOON_HIP(ctx, hipGetLastError());
+    return MOON_OK;
+}
+
+int launch_rotation_table(moon_ctx *ctx, float2 *table, size_t positions, size_t dims, double base, double factor) {
+    const size_t n = positions * (dims / 2);
+    if (!n) return MOON_OK;
+    hipLaunchKernelGGL(rotation_table_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, ctx->stream, table, n, (int)(dims / 2), base, factor);
     MOON_HIP(ctx, hipGetLastError());
     return MOON_OK;
 }

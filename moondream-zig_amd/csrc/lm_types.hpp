@@ -36,3 +36,4 @@ template <class T> __device__ __forceinline__ float dot_piece(const lm_u32x4 &w,
 // library exponentials: the gates and weights are wanted to f32 accuracy
 __device__ __forceinline__ float lm_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float lm_silu(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float lm_softcap(float z, float cap) { return cap * tanhf(z / cap); }

@@ -96,14 +96,15 @@ struct Fields { // typed access to a config's members; the first failure is kept
         }
         return (size_t)v->num;
     }
-    float number(const Json *j, const char *key, const std::string &where) {
+    double real(const Json *j, const char *key, const std::string &where) {
         const Json *v = j ? j->find(key) : nullptr;
         if (!v || v->type != Json::NUMBER) {
             fail(where + key + " is missing or no number");
-            return 1.0f;
+            return 1.0;
         }
-        return (float)v->num;
+        return v->num;
     }
+    float number(const Json *j, const char *key, const std::string &where) { return (float)real(j, key, where); }
 };
 
 std::string indexed(const char *prefix, size_t i, const std::string &rest) { return prefix + std::to_string(i) + rest; }
@@ -157,6 +158,95 @@ bool parse_rikanex(const Json &c, LayerListSpec *s, std::string *err) {
     return f.ok;
 }
 
+// Generax: parallel layers with RMS norms.  The mixer is windowed attention with rotated queries, keys and values, or windowed attention
+// without positions over tokens and pooled blocks beside a gated delta rule; the feed-forward is gated and dense.
+struct GeneraxReader {
+    Fields f;
+    const LayerListSpec *s;
+
+    void heads(const Json *m, const std::string &at, size_t *h, size_t *g, size_t *dim, size_t *vdim) {
+        *h = f.size(m, "heads", at);
+        *g = f.size(m, "kv_heads", at);
+        *dim = f.size(m, "dim", at);
+        *vdim = f.size(m, "vdim", at);
+        if (*h % *g) f.fail(at + "kv_heads does not divide heads");
+    }
+    // index of layer i, for kv_from
+    void attention(const Json *m, const std::string &at, size_t i, MixerSpec *x) {
+        heads(m, at, &x->heads, &x->kv_heads, &x->dim, &x->vdim);
+        x->scale = f.number(m, "scale", at);
+        x->qk_whole_norm = true;
+        const Json *mask = m ? m->find("mask") : nullptr;
+        if (mask && mask->type != Json::NIL) {
+            x->window = f.size(mask, "size", at + "mask.");
+            if (const Json *pool = mask->find("pool"); pool && pool->type != Json::NIL) x->pool = f.size(mask, "pool", at + "mask.");
+        }
+        const Json *rot = m ? m->find("rot") : nullptr;
+        if (rot && rot->type != Json::NIL) {
+            x->rot_dims = f.size(rot, "dims", at + "rot.");
+            x->rot_base = f.real(rot, "base", at + "rot.");
+            const Json *scaling = rot->find("scaling");
+            if (scaling && scaling->type != Json::NIL) x->rot_factor = f.real(scaling, "factor", at + "rot.scaling.");
+            x->rot_values = true;
+            if (x->rot_dims % 2 || x->rot_dims > x->dim) f.fail(at + "rot.dims is odd or exceeds dim");
+            if (x->vdim % 2) f.fail(at + "vdim is odd");
+            if (!(x->rot_base > 0.0) || !(x->rot_factor > 0.0)) f.fail(at + "rot.base and rot.scaling.factor must be positive");
+        }
+        const Json *from = m ? m->find("kv_from") : nullptr;
+        if (!from || from->type == Json::NIL) return;
+        if (!from->is_size() || from->num >= (double)i) {
+            f.fail(at + "kv_from is no earlier layer");
+            return;
+        }
+        x->kv_from = (int)from->num;
+        const LayerSpec &src = s->layers[x->kv_from];
+        const MixerSpec &y = src.mixer;
+        if (src.delta.heads || y.kv_from >= 0 || y.kv_heads != x->kv_heads || y.dim != x->dim || y.vdim != x->vdim || y.rot_dims != x->rot_dims ||
+            y.rot_base != x->rot_base || y.rot_factor != x->rot_factor || (x->pool && x->pool != y.pool))
+            f.fail(at + "kv_from names a layer without keys and values of its own, or of other heads or rotation");
+    }
+};
+bool parse_generax(const Json &c, LayerListSpec *s, std::string *err) {
+    GeneraxReader r{{err}, s};
+    Fields &f = r.f;
+    s->vocab = f.size(&c, "vocab", "");
+    s->width = f.size(&c, "width", "");
+    s->eps = f.number(f.object(c, "norm", ""), "eps", "norm.");
+    if (!(s->eps > 0.0f)) f.fail("norm.eps must be positive");
+    s->rms_norm = true;
+    if (const Json *cap = c.find("logit_softcap"); cap && cap->type != Json::NIL) {
+        s->softcap = f.number(&c, "logit_softcap", "");
+        if (!(s->softcap > 0.0f)) f.fail("logit_softcap must be positive");
+    }
+    const Json *layers = c.find("layers");
+    if (!layers || layers->type != Json::ARRAY || layers->items.empty()) return f.fail("layers is missing or empty");
+    for (size_t i = 0; i < layers->items.size() && f.ok; i++) {
+        const Json &l = layers->items[i];
+        const std::string at = "layers[" + std::to_string(i) + "].";
+        LayerSpec spec;
+        const Json *type = l.find("type"), *m = f.object(l, "mixer", at);
+        if (type && type->str == "attention") {
+            r.attention(m, at + "mixer.", i, &spec.mixer);
+            spec.mixer.temp = true;
+        } else if (type && type->str == "parallel") {
+            r.attention(m ? f.object(*m, "left", at + "mixer.") : nullptr, at + "mixer.left.", 0, &spec.mixer);
+            const std::string right = at + "mixer.right.";
+            const Json *d = m ? f.object(*m, "right", at + "mixer.") : nullptr;
+            r.heads(d, right, &spec.delta.heads, &spec.delta.kv_heads, &spec.delta.dim, &spec.delta.vdim);
+            spec.delta.conv = f.size(d, "conv", right);
+        } else return f.fail(at + "type is neither 'attention' nor 'parallel'");
+        const Json *mlp = l.find("mlp");
+        if (mlp && mlp->type != Json::NIL) {
+            const Json *kind = mlp->find("kind");
+            if (!kind || kind->str != "dense") return f.fail(at + "mlp.kind is not 'dense'");
+            spec.ff.kind = FeedForwardSpec::DENSE;
+            spec.ff.ff = f.size(mlp, "ff", at + "mlp.");
+        }
+        s->layers.push_back(spec);
+    }
+    return f.ok;
+}
+
 const TensorNames RIKANEX_NAMES = {
     [] { return std::string("embed"); },
     [] { return std::string("head"); },
@@ -167,9 +257,14 @@ const TensorNames RIKANEX_NAMES = {
     [](size_t i, size_t e, const char *what) { return indexed("l", i, indexed(".mlp.e", e, std::string(".") + what)); },
     ".b",
 };
+const TensorNames GENERAX_NAMES = {
+    RIKANEX_NAMES.embed, RIKANEX_NAMES.head, RIKANEX_NAMES.final_norm, RIKANEX_NAMES.norm, RIKANEX_NAMES.mixer, RIKANEX_NAMES.ff,
+    RIKANEX_NAMES.expert, nullptr, "left.", "right.",
+};
 
 const Design DESIGNS[] = {
     {"Rikanex", parse_rikanex, RIKANEX_NAMES},
+    {"Generax", parse_generax, GENERAX_NAMES},
 };
 
 } // namespace
@@ -220,32 +315,73 @@ int check_tensor(const SafeTensors &file, const std::string &name, std::initiali
 
 } // namespace
 
-// Every tensor of the description, with its shape
-static int check_tensors(const Design &design, const LayerListSpec &s, const SafeTensors &file, std::string *err) {
+// Every tensor of the description, with its shape.  Sizes that only the tensors have (the ranks of two-step projections) are taken
+// from them.
+static int check_tensors(const Design &design, LayerListSpec &s, const SafeTensors &file, std::string *err) {
     const TensorNames &n = design.names;
     const size_t w = s.width;
     int rc = MOON_OK;
     auto need = [&](const std::string &name, std::initializer_list<size_t> shape) {
         if (rc == MOON_OK) rc = check_tensor(file, name, shape, err);
     };
+    auto norm = [&](const std::string &name) {
+        need(name, {w});
+        if (n.bias_suffix) need(name + n.bias_suffix, {w});
+    };
     need(n.embed(), {s.vocab, w});
     need(n.head(), {s.vocab, w});
-    need(n.final_norm(), {w});
-    need(n.final_norm() + n.bias_suffix, {w});
+    norm(n.final_norm());
     bool mixing = false;
     for (size_t i = 0; i < s.layers.size() && rc == MOON_OK; i++) {
         const MixerSpec &m = s.layers[i].mixer;
+        DeltaSpec &d = s.layers[i].delta;
         const FeedForwardSpec &f = s.layers[i].ff;
-        need(n.norm(i), {w});
-        need(n.norm(i) + n.bias_suffix, {w});
-        need(n.mixer(i, "q"), {m.heads * m.dim, w});
-        need(n.mixer(i, "k"), {m.kv_heads * m.dim, w});
-        need(n.mixer(i, "v"), {m.kv_heads * m.vdim, w});
-        need(n.mixer(i, "o"), {w, m.heads * m.vdim});
-        if (m.gate) need(n.mixer(i, "g"), {m.heads * m.vdim, w});
-        if (m.sink) need(n.mixer(i, "sink"), {m.heads});
-        if (m.v_mix && mixing) need(n.mixer(i, "vmix"), {});
+        norm(n.norm(i));
+        auto mix = [&](const std::string &what) { return n.mixer(i, ((d.heads ? n.attention_part : "") + what).c_str()); };
+        need(mix("q"), {m.heads * m.dim, w});
+        if (m.kv_from < 0) {
+            need(mix("k"), {m.kv_heads * m.dim, w});
+            need(mix("v"), {m.kv_heads * m.vdim, w});
+        }
+        need(mix("o"), {w, m.heads * m.vdim});
+        if (m.qk_whole_norm) {
+            need(mix("q.norm"), {m.heads * m.dim});
+            if (m.kv_from < 0) need(mix("k.norm"), {m.kv_heads * m.dim});
+        }
+        if (m.temp) need(mix("temp"), {m.heads});
+        if (m.gate) need(mix("g"), {m.heads * m.vdim, w});
+        if (m.sink) need(mix("sink"), {m.heads});
+        if (m.v_mix && mixing) need(mix("vmix"), {});
         mixing = mixing || m.v_mix;
+        if (d.heads) {
+            auto delta = [&](const std::string &what) { return n.mixer(i, (n.delta_part + what).c_str()); };
+            auto rank = [&](const std::string &name, size_t *r) {
+                const StTensor *t = file.find(name);
+                if (t && t->shape.size() == 2) *r = t->shape[0];
+                if (rc == MOON_OK && t && (!*r || *r > 1 << 20)) {
+                    *err = "tensor '" + name + "' has no rows";
+                    rc = MOON_ESHAPE;
+                }
+                need(name, {*r, w});
+            };
+            const size_t q = d.kv_heads * d.dim, v = d.heads * d.vdim;
+            for (const char *what : {"q", "k", "v"}) {
+                const size_t rows = *what == 'v' ? v : q;
+                need(delta(what), {rows, w});
+                need(delta(what + std::string(".conv")), {rows, d.conv});
+            }
+            rank(delta("a1"), &d.rank_a);
+            rank(delta("g1"), &d.rank_g);
+            need(delta("a2"), {d.heads * d.dim, d.rank_a});
+            need(delta("g2"), {v, d.rank_g});
+            need(delta("b"), {d.heads, w});
+            need(delta("A_log"), {d.heads});
+            need(delta("dt_bias"), {d.heads * d.dim});
+            need(delta("norm"), {d.vdim});
+            need(delta("o"), {w, v});
+            need(mix("out"), {w});
+            need(delta("out"), {w});
+        }
         if (f.kind == FeedForwardSpec::DENSE) {
             need(n.ff(i, "gate"), {f.ff, w});
             need(n.ff(i, "up"), {f.ff, w});

@@ -31,10 +31,13 @@ struct SafeTensors {
 struct TensorNames {
     std::string (*embed)(), (*head)(), (*final_norm)();
     std::string (*norm)(size_t layer);
-    std::string (*mixer)(size_t layer, const char *what);            // q k v o g sink vmix
+    std::string (*mixer)(size_t layer, const char *what);            // q k v o g sink vmix q.norm k.norm temp; see also below
     std::string (*ff)(size_t layer, const char *what);               // gate up down router correction
     std::string (*expert)(size_t layer, size_t e, const char *what); // gate up down
     const char *bias_suffix;                                         // of a norm's bias
+    // where a mixer has a delta rule beside the attention: what comes before the names of each (the delta rule's are q k v, each with
+    // .conv, b A_log a1 a2 dt_bias g1 g2 norm o; out is the norm of each one's output)
+    const char *attention_part = "", *delta_part = "";
 };
 struct Design {
     const char *name; // config.json "architecture"

@@ -76,6 +76,7 @@ __device__ __forceinline__ void seg_store(const SegGemm &p, const float16_t (&ac
 #pragma unroll
                 for (int q = 0; q < 4; q++) {
                     float4 o = {acc[ni][mi][4 * q], acc[ni][mi][4 * q + 1], acc[ni][mi][4 * q + 2], acc[ni][mi][4 * q + 3]};
+                    if (p.softcap > 0.0f) o = {lm_softcap(o.x, p.softcap), lm_softcap(o.y, p.softcap), lm_softcap(o.z, p.softcap), lm_softcap(o.w, p.softcap)};
                     *reinterpret_cast<float4 *>(s + col * SEG_PITCH32 + ni * 32 + 8 * q + 4 * g) = o;
                 }
             asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -114,7 +115,7 @@ __global__ __launch_bounds__(DMA_THREADS) void seg_gemm_bf16_kernel(SegGemm p) {
     extern __shared__ __attribute__((aligned(16))) half_t lds_dma[]; // (the tile product addresses LDS from 0: nothing static beside it)
     TilePos t;
     if (!seg_tile(p, BM, BN, t)) return;
-    const int k_begin = t.split * p.k_per_split, k_end = min(p.K, k_begin + p.k_per_split), n_ktiles = (k_end - k_begin + BK - 1) / BK;
+    const int k_begin = p.kb[t.split], k_end = p.kb[t.split + 1], n_ktiles = (k_end - k_begin + BK - 1) / BK;
     if (n_ktiles <= 0) return;
     const int lane = threadIdx.x & 63, role_wave = (threadIdx.x >> 6) & 3;
     if (threadIdx.x >= 256) {
@@ -147,7 +148,7 @@ __global__ __launch_bounds__(256) void seg_gemm_f32_kernel(SegGemm p) {
     __shared__ float sa[F32_K][64 + 4], sw[F32_K][64 + 4];
     TilePos t;
     if (!seg_tile(p, SEG_TILE_ROWS, 64, t)) return;
-    const int k_begin = t.split * p.k_per_split, k_end = min(p.K, k_begin + p.k_per_split);
+    const int k_begin = p.kb[t.split], k_end = p.kb[t.split + 1];
     const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4, lr = tid >> 2, lk = (tid & 3) * 4;
     const float *A = reinterpret_cast<const float *>(p.A), *W = reinterpret_cast<const float *>(p.W) + size_t(t.group) * p.w_group;
     for (int mb = t.m0; mb < t.m_end; mb += 64) {
@@ -174,7 +175,7 @@ __global__ __launch_bounds__(256) void seg_gemm_f32_kernel(SegGemm p) {
             if (t.n0 < p.n16)
                 for (int j = 0; j < 4; j++) reinterpret_cast<float *>(p.c16)[size_t(m) * p.ld16 + t.n0 + tx + 16 * j] = acc[i][j];
             else if (t.n0 < p.n32)
-                for (int j = 0; j < 4; j++) p.c32[(size_t(t.split) * p.M + m) * p.ld32 + t.n0 - p.n16 + tx + 16 * j] = acc[i][j];
+                for (int j = 0; j < 4; j++) p.c32[(size_t(t.split) * p.M + m) * p.ld32 + t.n0 - p.n16 + tx + 16 * j] = p.softcap > 0.0f ? lm_softcap(acc[i][j], p.softcap) : acc[i][j];
             else
                 for (int j = 0; j < 2; j++)
                     reinterpret_cast<float *>(p.glu)[size_t(m) * p.ldg + (t.n0 - p.n32) / 2 + tx + 16 * j] = lm_silu(acc[i][j]) * acc[i][j + 2];
@@ -197,8 +198,12 @@ int launch_seg_gemm(moon_ctx *ctx, int dtype, SegGemm p) {
         return moon_fail(ctx, MOON_EINVAL_DIM, "segmented product: sizes must be padded to 64 (N %d, K %d, segments %d %d)", p.N, p.K, p.n16, p.n32);
     if (p.splits < 1) p.splits = 1;
     if (p.splits > 1 && (p.n16 || p.n32 != p.N || p.tile_group)) return moon_fail(ctx, MOON_EINVAL, "segmented product: only a plain f32 result splits k");
-    p.k_per_split = (int)pad_to((p.K + p.splits - 1) / p.splits, BK);
-    if ((p.splits - 1) * p.k_per_split >= p.K) return moon_fail(ctx, MOON_EINVAL, "segmented product: %d k splits leave one empty", p.splits);
+    if (p.splits > SEG_MAX_SPLITS) return moon_fail(ctx, MOON_EINVAL, "segmented product: %d k splits", p.splits);
+    if (!p.kb[p.splits])
+        for (int s = 0, per = (int)pad_to((p.K + p.splits - 1) / p.splits, BK); s <= p.splits; s++) p.kb[s] = std::min(p.K, s * per);
+    for (int s = 0; s < p.splits; s++)
+        if (p.kb[0] || p.kb[s] >= p.kb[s + 1] || p.kb[s + 1] % BK || p.kb[p.splits] != p.K)
+            return moon_fail(ctx, MOON_EINVAL, "segmented product: %d k splits leave one empty", p.splits);
     const int tile_n = dtype == MOON_DTYPE_BF16 ? BN : 64;
     const size_t tiles = size_t(p.tile_group ? p.max_tiles : (p.M + SEG_TILE_ROWS - 1) / SEG_TILE_ROWS) * ((p.N + tile_n - 1) / tile_n) * p.splits;
     const dim3 grid((unsigned)((tiles + 7) / 8 * 8));
