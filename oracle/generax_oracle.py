@@ -78,9 +78,9 @@ def attention(q, k, v, scale, window, pool=None):
     kb, vb = (pooled(k, pool), pooled(v, pool)) if pool else (k[:0], v[:0])
     out = np.zeros((T, H, v.shape[2]))
     for i in range(T):
-        js = [j for j in range(i + 1) if visible(i, j, window)]
-        bs = [b for b in range(len(kb)) if block_visible(i, b, window, pool)]
-        keys, values = np.concatenate([kb[bs], k[js]]), np.concatenate([vb[bs], v[js]])
+        lo = 0 if window is None else next(j for j in range(max(0, i - window - 1), i + 1) if visible(i, j, window))
+        n = next(b for b in range(max(0, (i - (window or 0)) // pool - 2), len(kb) + 1) if b == len(kb) or not block_visible(i, b, window, pool)) if pool else 0
+        keys, values = np.concatenate([kb[:n], k[lo:i + 1]]), np.concatenate([vb[:n], v[lo:i + 1]])
         for h in range(H):
             out[i, h] = softmax(keys[:, h // per] @ q[i, h] * scale[h]) @ values[:, h // per]
     return out

@@ -6,6 +6,7 @@ import sys
 import numpy as np
 import pytest
 import rikanex_oracle as R
+from decoder_checks import feed, opened, row_errors, rows_close, run
 from rikanex_models import (MODELS, ODD, TALL, WIDE, attention, config, dense, beacon_weights, layer, moe, tokens, weights, write_folder)
 
 pytestmark = pytest.mark.gpu
@@ -16,24 +17,17 @@ LIMIT = {"float32": 2e-5, "bfloat16": 3e-2}
 LENGTH = {"odd": 150, "wide": 300, "tall": 70}
 
 
-def row_errors(got, want):
-    return np.sqrt(((got - want) ** 2).mean(-1)) / np.sqrt((want**2).mean())
-
-
 # In bf16 a router's close call may fall the other way (in f32 none of these does): that many rows may be over the limit.
 FLIPS = {"float32": 0.0, "bfloat16": 0.03}
 
 
 def close(got, want, dtype, limit=None):
-    e = row_errors(got, want)
-    over = int((e > (limit or LIMIT[dtype])).sum())
-    ok = bool(np.isfinite(e).all() and over <= FLIPS[dtype] * len(e))
-    return ok, f"{dtype}: {over} of {len(e)} rows over the limit, worst {int(e.argmax())}: {e.max():.2e}"
+    return rows_close(got, want, limit or LIMIT[dtype], FLIPS[dtype])
 
 
 def assert_close(got, want, dtype, limit=None):
     ok, text = close(got, want, dtype, limit)
-    assert ok, text
+    assert ok, f"{dtype}: {text}"
 
 
 @pytest.fixture(scope="module")
@@ -45,27 +39,6 @@ def folders(tmp_path_factory):
         ids = tokens(LENGTH[name], cfg["vocab"])
         out[name] = (write_folder(tmp_path_factory.mktemp(name), cfg, w), cfg, w, ids, *R.forward(cfg, w, ids))
     return out
-
-
-def opened(moon, ctx, path, dtype, max_seq=512):
-    return moon.registry.open_text_model(str(path), dtype, max_seq, ctx)
-
-
-def run(moon, ctx, tmp_path, cfg, w, ids, dtype, portions=None, max_seq=512):
-    """Logits of all tokens, fed in portions (default: at once)."""
-    m = opened(moon, ctx, write_folder(tmp_path / "run", cfg, w), dtype, max_seq)
-    got = feed(m, ids, portions or [len(ids)])
-    m.close()
-    return got
-
-
-def feed(m, ids, portions):
-    out, at, i = [], 0, 0
-    while at < len(ids):
-        n = min(portions[i % len(portions)], len(ids) - at)
-        out.append(m.forward_logits(ids[at:at + n], np.arange(n)))
-        at, i = at + n, i + 1
-    return np.concatenate(out)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
