@@ -601,6 +601,39 @@ def bench_rikanex(moon, ctx, sizes, prompts=(768, 1920), steps=64):
     return out
 
 
+def generax_config(width, layers, heads, kv_heads, window, pool, ff):
+    """A Generax decoder with heads of 64: groups of two joined layers (attention over tokens and blocks beside a delta rule with as
+    many heads as the width holds), a layer of rotated attention and one that borrows its keys; or, with one ff, joined layers only."""
+    softmax = dict(heads=heads, kv_heads=kv_heads, dim=64, vdim=64, scale=0.125)
+    joined = dict(left=dict(softmax, mask=dict(size=window, pool=pool)), right=dict(heads=heads, kv_heads=heads, dim=64, vdim=64, conv=4))
+    turned = dict(softmax, mask=dict(size=window), rot=dict(dims=64, base=10000.0))
+    out = []
+    for i in range(layers):
+        kind = i % 4 if len(ff) == 3 else 0
+        mixer = joined if kind < 2 else turned if kind == 2 else dict(turned, kv_from=i - 1)
+        out.append(dict(type="parallel" if kind < 2 else "attention", mixer=mixer, mlp=dict(kind="dense", ff=ff[max(0, kind - 1)])))
+    return dict(architecture="Generax", vocab=V, width=width, norm=dict(eps=1e-5), logit_softcap=30.0, layers=out)
+
+
+# name -> (Generax configuration, the Rikanex decoder of equal width, layers, heads, window and layer bytes)
+GENERAX_SIZES = {
+    "w2048_l24_mixed": (generax_config(2048, 24, 32, 8, 1024, 16, (3712, 6464, 6848)), rikanex_config(2048, 24, 32, 8, 1024, ff=5824)),
+    "w2048_l24_joined": (generax_config(2048, 24, 32, 8, 1024, 16, (3712,)), rikanex_config(2048, 24, 32, 8, 1024, ff=5824)),
+    "w1024_l24_mixed": (generax_config(1024, 24, 16, 4, 512, 16, (1728, 3200, 3392)), rikanex_config(1024, 24, 16, 4, 512, ff=2816)),
+}
+
+
+def bench_generax(moon, ctx, sizes, prompts=(768, 1920), steps=64):
+    """Prefill and decode of the Generax decoder beside the Rikanex decoder of equal size (bf16, random weights), in one process."""
+    out = {}
+    for name in sizes:
+        for kind, cfg in zip(("generax", "rikanex"), GENERAX_SIZES[name]):
+            m = moon.text_model.TextModel.open_synthetic(cfg, "bfloat16", 2048, seed=0, std=0.02, ctx=ctx)
+            out.setdefault(name, {})[kind] = [time_decoder(ctx, m, n, steps) for n in prompts]
+            m.close()
+    return out
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -613,6 +646,8 @@ def main():
     ap.add_argument("--only-host-loops", action="store_true", help="only the host-stepped and operator-level decode legs")
     ap.add_argument("--rikanex", nargs="*", metavar="SIZE",
                     help="only the Rikanex decoder beside the f16 decoder of equal size, as its own JSON line (default: all of %s)" % ", ".join(RIKANEX_SIZES))
+    ap.add_argument("--generax", nargs="*", metavar="SIZE",
+                    help="only the Generax decoder beside the Rikanex decoder of equal size, as its own JSON line (default: all of %s)" % ", ".join(GENERAX_SIZES))
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="first run 8 plain 256 MiB copies (copy16_kernel) as the known-traffic yardstick for a counter run")
     ap.add_argument("--decode-mode", type=int, default=None,
@@ -623,8 +658,8 @@ def main():
     if PREFILL + args.warmup + args.steps + PROFILE_STEPS + 2 * SAMPLED_STEPS + 4 > 2048:
         sys.exit("bench.py: prefill 768 + warmup + steps + 32 profiled + 132 further steps must stay within the 2048-token KV cache")
 
-    for name in args.rikanex or []:
-        if name not in RIKANEX_SIZES:
+    for name, known in [(n, RIKANEX_SIZES) for n in args.rikanex or []] + [(n, GENERAX_SIZES) for n in args.generax or []]:
+        if name not in known:
             sys.exit(f"bench.py: unknown size {name}")
     moon = importlib.import_module("moondream-zig_amd")
     ctx = moon.Context(0)
@@ -643,6 +678,11 @@ def main():
         return
     if args.rikanex is not None:
         out = bench_rikanex(moon, ctx, args.rikanex or list(RIKANEX_SIZES))
+        ctx.close()
+        print(json.dumps(out))
+        return
+    if args.generax is not None:
+        out = bench_generax(moon, ctx, args.generax or list(GENERAX_SIZES))
         ctx.close()
         print(json.dumps(out))
         return

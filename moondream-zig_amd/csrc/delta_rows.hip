@@ -9,8 +9,8 @@
 //   delta_chunk   one workgroup per chunk and head: convolutions, unit vectors, decays, then A and P, and (I + A)^-1 applied to beta V
 //                 and beta K.  Quotients of decays are formed as products of the decays between the tokens, so nothing over- or underflows.
 //   delta_scan    one workgroup per head and 16 columns of the state, chunk after chunk: U = V' - K' S0, O, the new S, all with f32
-//                 matrix-core products (v_mfma_f32_16x16x4_f32: exact products, f32 sums).  The four wavefronts share the key channels;
-//                 an accumulator tile is the next product's second operand as it lies in the registers.
+//                 matrix-core products (v_mfma_f32_16x16x4_f32: f32 operands and sums).  Four wavefronts share the key channels; an
+//                 accumulator tile is the next product's second operand as it lies in the registers.
 //   delta_gate    RMS norm per head, weight, output gate.
 #include "delta_math.hpp"
 #include "lane_fold.hpp"
@@ -24,78 +24,116 @@ namespace {
 constexpr int DC = 16;      // tokens of a chunk
 constexpr int DC_PITCH = DC + 4;
 
-// One chunk and head in the scratch memory, in floats: K' [16][dimp], Q [16][dimp], R^T [dimp][16], G_15 [dimp], P [16][16], V' [16][vdimp]
+// One chunk and head in the scratch memory, in floats: K' [16][dimp], Q [16][dimp], R^T [dimp][16], G_15 [dimp], P [16][16], V'^T [vdimp][16]
 __host__ __device__ __forceinline__ size_t chunk_floats(int dimp, int vdimp) { return size_t(49) * dimp + 256 + size_t(16) * vdimp; }
 __host__ __device__ __forceinline__ size_t chunk_lds_floats(int dimp, int vdimp) {
     return size_t(3) * DC * (dimp + 16) + size_t(DC) * vdimp + 2 * DC * DC_PITCH + DC;
 }
 
+// Sixteen threads work on a token (and, for A and P, on a token s) until the columns are distributed.
 template <class T>
 __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaRows p) {
     extern __shared__ __attribute__((aligned(16))) float s_dc[];
     constexpr int PE = Piece<T>::N;
-    const int tid = threadIdx.x, lane = tid & 63, chunk = blockIdx.x / p.H, h = blockIdx.x % p.H, c = h / (p.H / p.G);
-    const int t0 = chunk * DC, cnt = min(DC, p.n - t0), dp = p.dimp + 16; // dp: row pitch
+    const int tid = threadIdx.x, lane = tid & 63, tok = tid >> 4, j = tid & 15, chunk = blockIdx.x / p.H, h = blockIdx.x % p.H, c = h / (p.H / p.G);
+    const int t0 = chunk * DC, dp = p.dimp + 16; // dp: row pitch
+    const bool there = t0 + tok < p.n; // tokens past the end are zero and decay nothing
     float *s_q = s_dc, *s_k = s_q + DC * dp, *s_g = s_k + DC * dp, *s_v = s_g + DC * dp, *s_a = s_v + DC * p.vdimp, *s_p = s_a + DC * DC_PITCH,
           *s_b = s_p + DC * DC_PITCH;
-    // convolutions, 16 bytes of channels at a time; tokens past the end are zero
-    const int pk = p.dimp / PE, pv = p.vdimp / PE, per_token = 2 * pk + pv;
+    // the decay's projection is requested before the convolutions' inputs
+    const float *dt = p.dt + size_t(t0 + (there ? tok : 0)) * p.lddt + h * p.dimp, *bias = p.dt_bias + h * p.dimp;
+    const int d_first = min(j * 4, p.dimp - 4);
+    const float4_t dt_first = *reinterpret_cast<const float4_t *>(dt + d_first) + *reinterpret_cast<const float4_t *>(bias + d_first);
+    const float rate = expf(p.a_log[h]), b_first = there ? p.beta[size_t(t0 + tok) * p.ldb + h] : 0.0f;
+    // convolutions, 16 bytes of channels at a time
+    constexpr int TAPS = 4; // inputs requested together
+    const int pk = p.dimp / PE, pieces = 2 * pk + p.vdimp / PE;
     const T *rows = reinterpret_cast<const T *>(p.c1) + p.oc, *ring = reinterpret_cast<const T *>(p.ring);
-    for (int i = tid; i < DC * per_token; i += 256) {
-        const int tok = i / per_token, piece = i % per_token, what = piece < pk ? 0 : piece < 2 * pk ? 1 : 2, off = (piece - what * pk) * PE;
+    for (int i = j; i < pieces; i += 16) {
+        const int what = (i >= pk) + (i >= 2 * pk), off = (i - what * pk) * PE;
         const int ch = (what == 0 ? c * p.dimp : what == 1 ? (p.G + c) * p.dimp : 2 * p.G * p.dimp + h * p.vdimp) + off;
         float acc[PE];
 #pragma unroll
         for (int e = 0; e < PE; e++) acc[e] = 0.0f;
-        if (tok < cnt)
-            for (int tap = 0; tap < p.taps; tap++) {
-                const int r = t0 + tok - (p.taps - 1) + tap, pos = p.pos0 + r;
-                if (pos < 0) continue;
-                float x[PE];
-                Piece<T>::unpack(*reinterpret_cast<const lm_u32x4 *>(r >= 0 ? rows + size_t(r) * p.ld + ch : ring + size_t(pos % p.taps) * p.channels + ch), x);
-                const float *w = p.conv + size_t(tap) * p.channels + ch;
+        if (there)
+            for (int tap0 = 0; tap0 < p.taps; tap0 += TAPS) {
+                lm_u32x4 x[TAPS];
 #pragma unroll
-                for (int e = 0; e < PE; e++) acc[e] = fmaf(w[e], x[e], acc[e]);
+                for (int u = 0; u < TAPS; u++) {
+                    const int r = t0 + tok - (p.taps - 1) + tap0 + u;
+                    x[u] = lm_u32x4{0, 0, 0, 0};
+                    if (tap0 + u >= p.taps) continue;
+                    if (r >= 0) x[u] = *reinterpret_cast<const lm_u32x4 *>(rows + size_t(r) * p.ld + ch);
+                    else if (p.pos0 + r >= 0) x[u] = *reinterpret_cast<const lm_u32x4 *>(ring + size_t((p.pos0 + r) % p.taps) * p.channels + ch);
+                }
+#pragma unroll
+                for (int u = 0; u < TAPS; u++) {
+                    if (tap0 + u >= p.taps) continue;
+                    float f[PE];
+                    Piece<T>::unpack(x[u], f);
+                    const float *w = p.conv + size_t(tap0 + u) * p.channels + ch;
+#pragma unroll
+                    for (int e = 0; e < PE; e++) acc[e] = fmaf(w[e], f[e], acc[e]);
+                }
             }
         float *dst = what == 0 ? s_q + tok * dp + off : what == 1 ? s_k + tok * dp + off : s_v + tok * p.vdimp + off;
 #pragma unroll
-        for (int e = 0; e < PE; e++) dst[e] = lm_silu(acc[e]);
+        for (int e = 0; e < PE; e += 4)
+            *reinterpret_cast<float4_t *>(dst + e) = float4_t{delta_silu(acc[e]), delta_silu(acc[e + 1]), delta_silu(acc[e + 2]), delta_silu(acc[e + 3])};
     }
-    for (int i = tid; i < DC * p.dimp; i += 256) {
-        const int tok = i / p.dimp, d = i % p.dimp;
-        s_g[tok * dp + d] = tok < cnt ? delta_decay(p.a_log[h], p.dt[size_t(t0 + tok) * p.lddt + h * p.dimp + d] + p.dt_bias[h * p.dimp + d]) : 1.0f;
-    }
-    if (tid < DC) s_b[tid] = tid < cnt ? lm_sigmoid(p.beta[size_t(t0 + tid) * p.ldb + h]) : 0.0f;
-    lds_barrier();
-    { // unit vectors: 8 lanes for each of the 32
-        float *x = (tid < 128 ? s_q : s_k) + (tid >> 3 & 15) * dp;
-        float ss = 0.0f;
-        for (int d = tid & 7; d < p.dimp; d += 8) ss = fmaf(x[d], x[d], ss);
+    for (int d = j * 4; d < p.dimp; d += 64) {
+        const float4_t z = d == j * 4 ? dt_first : *reinterpret_cast<const float4_t *>(dt + d) + *reinterpret_cast<const float4_t *>(bias + d);
+        float4_t g = {1.0f, 1.0f, 1.0f, 1.0f};
+        if (there)
 #pragma unroll
-        for (int off = 4; off >= 1; off >>= 1) ss += __shfl_xor(ss, off);
-        float f = 1.0f / sqrtf(ss + DELTA_UNIT_EPS);
-        if (tid < 128) f *= 1.0f / sqrtf((float)p.dim);
-        for (int d = tid & 7; d < p.dimp; d += 8) x[d] *= f;
+            for (int e = 0; e < 4; e++) g[e] = delta_decay(rate, z[e]);
+        *reinterpret_cast<float4_t *>(s_g + tok * dp + d) = g;
+    }
+    if (j == 0) s_b[tok] = there ? lm_sigmoid(b_first) : 0.0f;
+    { // unit vectors (a token's threads are in one wavefront, whose LDS accesses stay in order)
+        float *q = s_q + tok * dp, *k = s_k + tok * dp, ss_q = 0.0f, ss_k = 0.0f;
+        for (int d = j * 4; d < p.dimp; d += 64) {
+            const float4_t a = *reinterpret_cast<const float4_t *>(q + d), b = *reinterpret_cast<const float4_t *>(k + d);
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                ss_q = fmaf(a[e], a[e], ss_q);
+                ss_k = fmaf(b[e], b[e], ss_k);
+            }
+        }
+#pragma unroll
+        for (int off = 8; off >= 1; off >>= 1) {
+            ss_q += __shfl_xor(ss_q, off);
+            ss_k += __shfl_xor(ss_k, off);
+        }
+        const float f_q = 1.0f / (sqrtf(ss_q + DELTA_UNIT_EPS) * sqrtf((float)p.dim)), f_k = 1.0f / sqrtf(ss_k + DELTA_UNIT_EPS);
+        for (int d = j * 4; d < p.dimp; d += 64) {
+            *reinterpret_cast<float4_t *>(q + d) *= f_q;
+            *reinterpret_cast<float4_t *>(k + d) *= f_k;
+        }
     }
     lds_barrier();
-    { // A and P: a thread has token s and every 16th channel
-        const int s = tid >> 4;
+    { // A and P: a thread has token s = tok and four of every 64 channels
         float v[2 * DC];
 #pragma unroll
         for (int i = 0; i < 2 * DC; i++) v[i] = 0.0f;
-        for (int d = tid & 15; d < p.dimp; d += 16) {
-            float w = s_k[s * dp + d]; // k_s times the decays of the tokens behind s up to t
+        for (int d = j * 4; d < p.dimp; d += 64) {
+            const float4_t ks = *reinterpret_cast<const float4_t *>(s_k + tok * dp + d);
+            float4_t w = {0, 0, 0, 0}; // k_s times the decays of the tokens behind s up to t
 #pragma unroll
             for (int t = 0; t < DC; t++) {
-                if (t > s) w *= s_g[t * dp + d];
-                const float on = t >= s ? w : 0.0f;
-                v[t] = fmaf(s_k[t * dp + d], on, v[t]);
-                v[DC + t] = fmaf(s_q[t * dp + d], on, v[DC + t]);
+                const float4_t g = *reinterpret_cast<const float4_t *>(s_g + t * dp + d), k = *reinterpret_cast<const float4_t *>(s_k + t * dp + d),
+                               q = *reinterpret_cast<const float4_t *>(s_q + t * dp + d);
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    w[e] = t == tok ? ks[e] : w[e] * g[e];
+                    v[t] = fmaf(k[e], w[e], v[t]);
+                    v[DC + t] = fmaf(q[e], w[e], v[DC + t]);
+                }
             }
         }
         fold_lanes<2 * DC, 8>(v, lane, 1, 0, [&](int i, float x) {
-            if (i < DC) s_a[i * DC_PITCH + s] = i > s ? s_b[i] * x : 0.0f;
-            else s_p[(i - DC) * DC_PITCH + s] = x;
+            if (i < DC) s_a[i * DC_PITCH + tok] = i > tok ? s_b[i] * x : 0.0f;
+            else s_p[(i - DC) * DC_PITCH + tok] = x;
         });
     }
     lds_barrier();
@@ -103,6 +141,10 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaRows p) {
     float *o_k = out, *o_q = o_k + DC * p.dimp, *o_r = o_q + DC * p.dimp, *o_g = o_r + DC * p.dimp, *o_p = o_g + p.dimp, *o_v = o_p + DC * DC;
     for (int i = tid; i < 2 * p.dimp + p.vdimp; i += 256) {
         float x[DC];
+        auto store16 = [&](float *dst) {
+#pragma unroll
+            for (int t = 0; t < DC; t += 4) *reinterpret_cast<float4_t *>(dst + t) = float4_t{x[t], x[t + 1], x[t + 2], x[t + 3]};
+        };
         if (i < p.dimp + p.vdimp) { // a column of beta K or beta V, forward substitution
             const bool is_k = i < p.dimp;
             const float *src = is_k ? s_k + i : s_v + i - p.dimp, *g = s_g + i;
@@ -113,13 +155,17 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaRows p) {
                 if (is_k) all *= g[t * dp];
                 float y = s_b[t] * src[t * pitch] * all;
 #pragma unroll
-                for (int s = 0; s < t; s++) y = fmaf(-s_a[t * DC_PITCH + s], x[s], y);
+                for (int s0 = 0; s0 < t; s0 += 4) {
+                    const float4_t a = *reinterpret_cast<const float4_t *>(s_a + t * DC_PITCH + s0);
+#pragma unroll
+                    for (int s = s0; s < t && s < s0 + 4; s++) y = fmaf(-a[s - s0], x[s], y);
+                }
                 x[t] = y;
             }
-            float *dst = is_k ? o_k + i : o_v + i - p.dimp;
-            const int ld = is_k ? p.dimp : p.vdimp;
+            if (is_k) {
 #pragma unroll
-            for (int t = 0; t < DC; t++) dst[size_t(t) * ld] = x[t];
+                for (int t = 0; t < DC; t++) o_k[size_t(t) * p.dimp + i] = x[t];
+            } else store16(o_v + size_t(i - p.dimp) * DC);
         } else { // Q, R and the whole chunk's decay
             const int d = i - p.dimp - p.vdimp;
             float all = 1.0f, rest = 1.0f;
@@ -133,25 +179,72 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaRows p) {
                 x[t] = s_k[t * dp + d] * rest;
                 rest *= s_g[t * dp + d];
             }
-#pragma unroll
-            for (int t = 0; t < DC; t += 4) *reinterpret_cast<float4 *>(o_r + size_t(d) * DC + t) = float4{x[t], x[t + 1], x[t + 2], x[t + 3]};
+            store16(o_r + size_t(d) * DC);
             o_g[d] = all;
         }
     }
     o_p[tid] = s_p[(tid >> 4) * DC_PITCH + (tid & 15)];
 }
 
-// NT: tiles of 16 key channels a wavefront owns; AHEAD: chunks whose operands are requested before they are needed
+// Four wavefronts share the key channels, NT tiles of 16 each; the fifth one finishes the outputs, a chunk behind.  AHEAD: chunks whose
+// operands are requested before they are needed.
+constexpr int SCAN_THREADS = 320;
 template <int NT> struct ScanChunk {
-    float4_t k[NT], q[NT], r[NT], g[NT], p, v;
+    float4_t k[NT], q[NT], r[NT], g[NT], v;
 };
 template <class T, int NT, int AHEAD>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void delta_scan_kernel(DeltaRows p) {
+__global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_scan_kernel(DeltaRows p) {
     __shared__ float4_t s_u[2][4][64], s_o[2][4][64];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, quad = lane >> 4;
-    const int slices = p.vdimp / 16, h = blockIdx.x / slices, v0 = blockIdx.x % slices * 16, tiles = p.dimp / 16, chunks = (p.n + DC - 1) / DC;
+    const int slices = p.vdimp / 16, tiles = p.dimp / 16, chunks = (p.n + DC - 1) / DC;
+    // Workgroups are dealt to the eight dies round robin: a head's columns stay on the die whose L2 has its chunks (delta_chunk's mapping).
+    int h = blockIdx.x / slices, v0 = blockIdx.x % slices * 16;
+    if (p.H % 8 == 0) {
+        h = blockIdx.x / 8 / slices * 8 + blockIdx.x % 8;
+        v0 = blockIdx.x / 8 % slices * 16;
+    }
     const size_t stride = chunk_floats(p.dimp, p.vdimp);
     const float *src = p.scratch + size_t(h) * chunks * stride;
+    if (wave == 4) {
+        const size_t at_p = size_t(49) * p.dimp;
+        float4_t P[AHEAD], V[AHEAD], u_before, p_before;
+        auto request = [&](int a, int chunk) {
+            const float *ap = src + min(chunk, chunks - 1) * stride + at_p;
+            P[a] = *reinterpret_cast<const float4_t *>(ap + col * DC + 4 * quad);
+            V[a] = *reinterpret_cast<const float4_t *>(ap + (DC + v0 + col) * DC + 4 * quad);
+        };
+        auto finish = [&](int chunk, int half) { // chunk's parts lie in `half`
+            float4_t o = (s_o[half][0][lane] + s_o[half][1][lane]) + (s_o[half][2][lane] + s_o[half][3][lane]);
+#pragma unroll
+            for (int j = 0; j < 4; j++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(p_before[j], u_before[j], o, 0, 0, 0);
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const int row = chunk * DC + 4 * quad + e;
+                if (row < p.n) p.o[(size_t(row) * p.H + h) * p.vdimp + v0 + col] = o[e];
+            }
+        };
+#pragma unroll
+        for (int a = 0; a < AHEAD; a++) request(a, a);
+        auto step = [&](int a, int chunk) {
+            const int half = chunk & 1;
+            lds_barrier();
+            const float4_t u = V[a] - ((s_u[half][0][lane] + s_u[half][1][lane]) + (s_u[half][2][lane] + s_u[half][3][lane]));
+            if (chunk) finish(chunk - 1, half);
+            u_before = u;
+            p_before = P[a];
+            request(a, chunk + AHEAD);
+        };
+        int base = 0;
+        for (; base + AHEAD <= chunks; base += AHEAD)
+#pragma unroll
+            for (int a = 0; a < AHEAD; a++) step(a, base + a);
+#pragma unroll
+        for (int a = 0; a < AHEAD; a++)
+            if (base + a < chunks) step(a, base + a);
+        lds_barrier();
+        finish(chunks - 1, chunks & 1);
+        return;
+    }
     float *state = p.state + size_t(h) * p.dimp * p.vdimp + v0 + col;
     float4_t S[NT]; // rows 16 tile + 4 quad + e of column v0 + col
 #pragma unroll
@@ -166,58 +259,53 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void d
         const float *at = src + min(chunk, chunks - 1) * stride;
 #pragma unroll
         for (int i = 0; i < NT; i++) {
-            const int tile = wave + 4 * i;
-            if (tile < tiles) {
-                b.k[i] = *reinterpret_cast<const float4_t *>(at + col * p.dimp + 16 * tile + 4 * quad);
-                b.q[i] = *reinterpret_cast<const float4_t *>(at + (DC + col) * p.dimp + 16 * tile + 4 * quad);
-                b.r[i] = *reinterpret_cast<const float4_t *>(at + 2 * DC * p.dimp + (16 * tile + col) * DC + 4 * quad);
-                b.g[i] = *reinterpret_cast<const float4_t *>(at + 3 * DC * p.dimp + 16 * tile + 4 * quad);
-            } else b.k[i] = b.q[i] = b.r[i] = b.g[i] = float4_t{0, 0, 0, 0};
+            const int tile = min(wave + 4 * i, tiles - 1);
+            b.k[i] = *reinterpret_cast<const float4_t *>(at + col * p.dimp + 16 * tile + 4 * quad);
+            b.q[i] = *reinterpret_cast<const float4_t *>(at + (DC + col) * p.dimp + 16 * tile + 4 * quad);
+            b.r[i] = *reinterpret_cast<const float4_t *>(at + 2 * DC * p.dimp + (16 * tile + col) * DC + 4 * quad);
+            b.g[i] = *reinterpret_cast<const float4_t *>(at + 3 * DC * p.dimp + 16 * tile + 4 * quad);
         }
-        const float *ap = at + size_t(49) * p.dimp;
-        b.p = *reinterpret_cast<const float4_t *>(ap + col * DC + 4 * quad);
-#pragma unroll
-        for (int e = 0; e < 4; e++) b.v[e] = ap[DC * DC + (4 * quad + e) * p.vdimp + v0 + col];
+        b.v = *reinterpret_cast<const float4_t *>(at + size_t(49) * p.dimp + (DC + v0 + col) * DC + 4 * quad);
     };
 #pragma unroll
     for (int a = 0; a < AHEAD; a++) request(ring[a], a);
-    for (int base = 0; base < chunks; base += AHEAD) {
+    float4_t o = {0, 0, 0, 0};
+    auto step = [&](ScanChunk<NT> &b, int chunk) {
+        const int half = chunk & 1;
+        float4_t u = {0, 0, 0, 0};
 #pragma unroll
-        for (int a = 0; a < AHEAD; a++) {
-            const int chunk = base + a;
-            if (chunk >= chunks) break; // (the same in every wavefront)
-            ScanChunk<NT> &b = ring[a];
-            float4_t u = {0, 0, 0, 0}, o = {0, 0, 0, 0};
+        for (int i = 0; i < NT; i++) // (a tile past the end is another wavefront's, with a state of zero here)
 #pragma unroll
-            for (int i = 0; i < NT; i++)
+            for (int j = 0; j < 4; j++) u = __builtin_amdgcn_mfma_f32_16x16x4f32(b.k[i][j], S[i][j], u, 0, 0, 0);
+        s_u[half][wave][lane] = u;
+        s_o[half][wave][lane] = o; // (of the chunk before)
+        lds_barrier(); // (one per chunk: what a chunk reads is written again two chunks later)
+        const float4_t u0 = s_u[half][0][lane], u1 = s_u[half][1][lane], u2 = s_u[half][2][lane], u3 = s_u[half][3][lane];
+        o = float4_t{0, 0, 0, 0};
 #pragma unroll
-                for (int j = 0; j < 4; j++) {
-                    u = __builtin_amdgcn_mfma_f32_16x16x4f32(b.k[i][j], S[i][j], u, 0, 0, 0);
-                    o = __builtin_amdgcn_mfma_f32_16x16x4f32(b.q[i][j], S[i][j], o, 0, 0, 0);
-                }
-            s_u[chunk & 1][wave][lane] = u;
-            s_o[chunk & 1][wave][lane] = o;
-            lds_barrier(); // (one per chunk: what a chunk reads is written again two chunks later)
-            u = b.v - ((s_u[chunk & 1][0][lane] + s_u[chunk & 1][1][lane]) + (s_u[chunk & 1][2][lane] + s_u[chunk & 1][3][lane]));
+        for (int i = 0; i < NT; i++)
 #pragma unroll
-            for (int i = 0; i < NT; i++) {
-                S[i] *= b.g[i];
+            for (int j = 0; j < 4; j++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(b.q[i][j], S[i][j], o, 0, 0, 0);
+        u = b.v - ((u0 + u1) + (u2 + u3));
 #pragma unroll
-                for (int j = 0; j < 4; j++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(b.r[i][j], u[j], S[i], 0, 0, 0);
-            }
-            if (wave == (chunk & 3)) {
-                o = (s_o[chunk & 1][0][lane] + s_o[chunk & 1][1][lane]) + (s_o[chunk & 1][2][lane] + s_o[chunk & 1][3][lane]);
+        for (int i = 0; i < NT; i++) {
+            S[i] *= b.g[i];
 #pragma unroll
-                for (int j = 0; j < 4; j++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(b.p[j], u[j], o, 0, 0, 0);
-#pragma unroll
-                for (int e = 0; e < 4; e++) {
-                    const int row = chunk * DC + 4 * quad + e;
-                    if (row < p.n) p.o[(size_t(row) * p.H + h) * p.vdimp + v0 + col] = o[e];
-                }
-            }
-            if (chunk + AHEAD < chunks) request(b, chunk + AHEAD);
+            for (int j = 0; j < 4; j++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(b.r[i][j], u[j], S[i], 0, 0, 0);
+            if (wave + 4 * i >= tiles) S[i] = float4_t{0, 0, 0, 0};
         }
-    }
+        request(b, chunk + AHEAD);
+    };
+    // (no exit inside the rounds: with one, every wait for a chunk's operands would also wait for the ones requested last)
+    int base = 0;
+    for (; base + AHEAD <= chunks; base += AHEAD)
+#pragma unroll
+        for (int a = 0; a < AHEAD; a++) step(ring[a], base + a);
+#pragma unroll
+    for (int a = 0; a < AHEAD; a++)
+        if (base + a < chunks) step(ring[a], base + a);
+    s_o[chunks & 1][wave][lane] = o;
+    lds_barrier();
 #pragma unroll
     for (int i = 0; i < NT; i++)
 #pragma unroll
@@ -272,10 +360,10 @@ template <class T> int delta_launch(moon_ctx *ctx, const DeltaRows &p) {
     MOON_HIP(ctx, hipGetLastError());
     const dim3 grid((unsigned)(p.vdimp / 16) * p.H);
     const int nt = (p.dimp / 16 + 3) / 4;
-    if (nt <= 1) hipLaunchKernelGGL((delta_scan_kernel<T, 1, 4>), grid, dim3(256), 0, ctx->stream, p);
-    else if (nt <= 2) hipLaunchKernelGGL((delta_scan_kernel<T, 2, 4>), grid, dim3(256), 0, ctx->stream, p);
-    else if (nt <= 4) hipLaunchKernelGGL((delta_scan_kernel<T, 4, 2>), grid, dim3(256), 0, ctx->stream, p);
-    else hipLaunchKernelGGL((delta_scan_kernel<T, 8, 1>), grid, dim3(256), 0, ctx->stream, p);
+    if (nt <= 1) hipLaunchKernelGGL((delta_scan_kernel<T, 1, 8>), grid, dim3(SCAN_THREADS), 0, ctx->stream, p);
+    else if (nt <= 2) hipLaunchKernelGGL((delta_scan_kernel<T, 2, 4>), grid, dim3(SCAN_THREADS), 0, ctx->stream, p);
+    else if (nt <= 4) hipLaunchKernelGGL((delta_scan_kernel<T, 4, 2>), grid, dim3(SCAN_THREADS), 0, ctx->stream, p);
+    else hipLaunchKernelGGL((delta_scan_kernel<T, 8, 1>), grid, dim3(SCAN_THREADS), 0, ctx->stream, p);
     MOON_HIP(ctx, hipGetLastError());
     int lph = 1;
     while (lph < p.vdimp / 4 && lph < 64) lph *= 2;

@@ -285,17 +285,39 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
         pv[i] = lm_u32x4{0, 0, 0, 0};
         if (key < j1 && key != newest && vc0 < vp) pv[i] = v_piece(key, vc0);
     }
-    float f_q = 1.0f, f_k = 1.0f;
-    if (WHOLE && p.whole) { // q and k are normed as a whole
+    // element d of a head x, times its weight w, turned by its pair's angle
+    auto turned = [&](const float *x, const float *w, int d, const float2 *table, int half) {
+        float y = w ? x[d] * w[d] : x[d];
+        if (!table || d >= 2 * half) return y;
+        const int m = d < half ? d : d - half, other = d < half ? d + half : m;
+        const float2 cs = table[size_t(pos) * half + m];
+        const float z = w ? x[other] * w[other] : x[other];
+        return d < half ? y * cs.x - z * cs.y : y * cs.x + z * cs.y;
+    };
+    // where the outputs turn back: the angle of this thread's first element, requested early
+    const int back = WHOLE && p.rotv ? p.vdim / 2 : 0;
+    float2 back_cs = {1.0f, 0.0f};
+    if (WHOLE && back && tid % p.vdimp < 2 * back) back_cs = p.rotv[size_t(pos) * back + tid % p.vdimp % back];
+    if constexpr (WHOLE) {
+        // q and k are normed as a whole: the heads go to LDS turned and weighted, the norms' factors come last
         float ss[2] = {0.0f, 0.0f};
         const int nq = p.H * p.dimp, nk = has_new ? p.G * p.dimp : 0;
-        for (int i = tid * 4; i < nq; i += 1024) {
-            const float4_t v = *reinterpret_cast<const float4_t *>(p.proj + i);
-            ss[0] += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+        if (p.whole) {
+            for (int i = tid * 4; i < nq; i += 1024) {
+                const float4_t v = *reinterpret_cast<const float4_t *>(p.proj + i);
+                ss[0] += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+            }
+            for (int i = tid * 4; i < nk; i += 1024) {
+                const float4_t v = *reinterpret_cast<const float4_t *>(p.proj + p.ok + i);
+                ss[1] += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+            }
         }
-        for (int i = tid * 4; i < nk; i += 1024) {
-            const float4_t v = *reinterpret_cast<const float4_t *>(p.proj + p.ok + i);
-            ss[1] += (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+        for (int task = wave; task < nh + (has_new ? 2 : 0); task += 4) {
+            const bool is_v = task == nh + 1, is_q = task < nh;
+            const float *src = p.proj + (is_v ? p.ov + g * p.vdimp : is_q ? (h0 + task) * p.dimp : p.ok + g * p.dimp);
+            const float *w = is_v || !p.whole ? nullptr : is_q ? p.qn + (h0 + task) * p.dimp : p.kn + g * p.dimp;
+            for (int d = lane; d < (is_v ? p.vdimp : p.dimp); d += 64)
+                (is_v ? s_v : is_q ? s_q + task * p.dimp : s_k)[d] = turned(src, w, d, is_v ? p.rotv : p.rot, (is_v ? p.vdim : p.rot_dims) / 2);
         }
         ss[0] = wave_sum(ss[0]);
         ss[1] = wave_sum(ss[1]);
@@ -304,23 +326,23 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
             s_r[2 * wave + 1] = ss[1];
         }
         lds_barrier();
-        f_q = 1.0f / sqrtf(((s_r[0] + s_r[2]) + (s_r[4] + s_r[6])) / (float)(p.H * p.dim) + p.eps);
-        f_k = 1.0f / sqrtf(((s_r[1] + s_r[3]) + (s_r[5] + s_r[7])) / (float)(p.G * p.dim) + p.eps);
-    }
-    // element d of a head x of `size` elements, times f and its weight w, turned by its pair's angle
-    auto turned = [&](const float *x, float f, const float *w, int d, const float2 *table, int half) {
-        float y = w ? x[d] * f * w[d] : x[d] * f;
-        if (!table || d >= 2 * half) return y;
-        const int m = d < half ? d : d - half, other = d < half ? d + half : m;
-        const float2 cs = table[size_t(pos) * half + m];
-        const float z = w ? x[other] * f * w[other] : x[other] * f;
-        return d < half ? y * cs.x - z * cs.y : y * cs.x + z * cs.y;
-    };
+        const float f_q = p.whole ? 1.0f / sqrtf(((s_r[0] + s_r[2]) + (s_r[4] + s_r[6])) / (float)(p.H * p.dim) + p.eps) : 1.0f;
+        const float f_k = p.whole ? 1.0f / sqrtf(((s_r[1] + s_r[3]) + (s_r[5] + s_r[7])) / (float)(p.G * p.dim) + p.eps) : 1.0f;
+        for (int i = tid; i < nh * p.dimp; i += 256) s_q[i] = (float)(T)(s_q[i] * f_q);
+        if (has_new)
+            for (int i = tid; i < p.dimp + p.vdimp; i += 256) {
+                const bool is_v = i >= p.dimp;
+                const int d = is_v ? i - p.dimp : i;
+                const T c = (T)(is_v ? s_v[d] : s_k[d] * f_k);
+                (is_v ? s_v : s_k)[d] = (float)c;
+                if (hb == 0) (is_v ? cv + size_t(pos % p.cap) * p.vdimp : ck + size_t(pos % p.cap) * p.dimp)[d] = c;
+            }
+    } else
     for (int task = wave; task < nh + (has_new ? 2 : 0); task += 4) {
         if (task == nh + 1) { // the new value
             const T *first = p.mixes ? reinterpret_cast<const T *>(p.v_first) + (size_t(g) * p.cap_first + pos % p.cap_first) * p.vdimp : nullptr;
             for (int d = lane; d < p.vdimp; d += 64) {
-                float v = WHOLE && p.rotv ? turned(p.proj + p.ov + g * p.vdimp, 1.0f, nullptr, d, p.rotv, p.vdim / 2) : (float)(T)p.proj[p.ov + g * p.vdimp + d];
+                float v = (float)(T)p.proj[p.ov + g * p.vdimp + d];
                 if (first) v = (1.0f - p.lambda) * v + p.lambda * (float)first[d];
                 const T c = (T)v;
                 s_v[d] = (float)c;
@@ -332,9 +354,8 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
             float ss = 0.0f;
             for (int d = lane; d < p.dimp; d += 64) ss = fmaf(src[d], src[d], ss);
             const float f = p.qk_rms ? 1.0f / sqrtf(wave_sum(ss) / (float)p.dim + p.eps) : 1.0f;
-            const float *w = is_q ? p.qn + (h0 + task) * p.dimp : p.kn + g * p.dimp;
             for (int d = lane; d < p.dimp; d += 64) {
-                const T c = (T)(WHOLE ? turned(src, is_q ? f_q : f_k, p.whole ? w : nullptr, d, p.rot, p.rot_dims / 2) : src[d] * f);
+                const T c = (T)(src[d] * f);
                 if (is_q) s_q[task * p.dimp + d] = (float)c;
                 else {
                     s_k[d] = (float)c;
@@ -519,12 +540,11 @@ __device__ __forceinline__ void mix_attention(const DecodeMix &p, int g, int hb,
     if (!(WHOLE && p.rotv)) return;
     lds_barrier();
     for (int i = tid; i < nh * p.vdimp; i += 256) { // the outputs turn back
-        const int h = i / p.vdimp, d = i % p.vdimp, half = p.vdim / 2;
+        const int h = i / p.vdimp, d = i % p.vdimp;
         float o = s_o[i];
-        if (d < 2 * half) {
-            const int m = d < half ? d : d - half;
-            const float2 cs = p.rotv[size_t(pos) * half + m];
-            o = d < half ? o * cs.x + s_o[i + half] * cs.y : o * cs.x - s_o[i - half] * cs.y;
+        if (d < 2 * back) {
+            const float2 cs = i == tid ? back_cs : p.rotv[size_t(pos) * back + d % back];
+            o = d < back ? o * cs.x + s_o[i + back] * cs.y : o * cs.x - s_o[i - back] * cs.y;
         }
         if (p.gate) o *= lm_sigmoid(p.proj[p.og + (h0 + h) * p.vdimp + d]);
         reinterpret_cast<T *>(p.out)[(h0 + h) * p.vdimp + d] = (T)o;
@@ -563,12 +583,12 @@ __device__ __forceinline__ void mix_delta(const DecodeMix &p, int h, float *lds)
             const int at = pos - (p.taps - 1) + tap;
             if (at >= 0) acc = fmaf(p.conv[size_t(tap) * p.channels + ch], (float)ring[size_t(at % p.taps) * p.channels + ch], acc);
         }
-        acc = lm_silu(fmaf(p.conv[size_t(p.taps - 1) * p.channels + ch], (float)now, acc));
+        acc = delta_silu(fmaf(p.conv[size_t(p.taps - 1) * p.channels + ch], (float)now, acc));
         (i < dimp ? s_q + i : i < 2 * dimp ? s_k + i - dimp : s_v + i - 2 * dimp)[0] = acc;
         if (keep && (i >= 2 * dimp || h % per == 0)) reinterpret_cast<T *>(p.ring)[size_t(pos % p.taps) * p.channels + ch] = now; // (no tap reads this row)
     }
     for (int i = tid; i < p.kd; i += 256) s_in[i] = i < p.rank_a + p.rank_g ? (T)p.proj[p.od + i] : (T)0.0f;
-    const float beta = lm_sigmoid(p.beta[h]);
+    const float beta = lm_sigmoid(p.beta[h]), rate = expf(p.a_log[h]);
     lds_barrier();
     if (wave < 2) { // unit vectors
         float *x = wave ? s_k : s_q, ss = 0.0f;
@@ -579,20 +599,31 @@ __device__ __forceinline__ void mix_delta(const DecodeMix &p, int h, float *lds)
     }
     { // second steps of the decay's and the gate's projections, 8 lanes a row
         const int a_end = (p.rank_a + PE - 1) / PE, g_begin = p.rank_a / PE, g_end = (p.rank_a + p.rank_g + PE - 1) / PE, rows = dimp + vdimp;
-#pragma unroll 4
-        for (int i = tid >> 3; i < (rows + 31) / 32 * 32; i += 32) {
-            const bool is_a = i < dimp;
-            float acc = 0.0f;
-            if (i < rows) {
+        constexpr int RU = 4; // rows a lane works on at a time
+        for (int base = tid >> 3; base < (rows + 31) / 32 * 32; base += 32 * RU) {
+            float acc[RU];
+#pragma unroll
+            for (int u = 0; u < RU; u++) {
+                const int i = base + 32 * u;
+                const bool is_a = i < dimp;
+                acc[u] = 0.0f;
+                if (i >= rows) continue;
                 const T *w = reinterpret_cast<const T *>(p.wlr) + size_t(is_a ? p.lr16 + h * dimp + i : h * vdimp + i - dimp) * p.kd;
-                for (int q = (is_a ? 0 : g_begin) + (tid & 7); q < (is_a ? a_end : g_end); q += 8) // (the other step's columns are zero)
-                    acc = dot_piece<T>(reinterpret_cast<const lm_u32x4 *>(w)[q], *reinterpret_cast<const lm_u32x4 *>(s_in + q * PE), acc);
+                const int end = is_a ? a_end : g_end, first = (is_a ? 0 : g_begin) + (tid & 7); // (the other step's columns are zero)
+                for (int q = first; q < end; q += 8)
+                    acc[u] = dot_piece<T>(reinterpret_cast<const lm_u32x4 *>(w)[q], *reinterpret_cast<const lm_u32x4 *>(s_in + q * PE), acc[u]);
             }
 #pragma unroll
-            for (int off = 4; off >= 1; off >>= 1) acc += __shfl_xor(acc, off);
-            if ((tid & 7) || i >= rows) continue;
-            if (is_a) s_g[i] = delta_decay(p.a_log[h], acc + p.dt_bias[h * dimp + i]);
-            else s_gate[i - dimp] = lm_sigmoid(acc);
+            for (int off = 4; off >= 1; off >>= 1)
+#pragma unroll
+                for (int u = 0; u < RU; u++) acc[u] += __shfl_xor(acc[u], off);
+#pragma unroll
+            for (int u = 0; u < RU; u++) {
+                const int i = base + 32 * u;
+                if ((tid & 7) || i >= rows) continue;
+                if (i < dimp) s_g[i] = delta_decay(rate, acc[u] + p.dt_bias[h * dimp + i]);
+                else s_gate[i - dimp] = lm_sigmoid(acc[u]);
+            }
         }
     }
     lds_barrier();
@@ -844,6 +875,7 @@ int launch_decode_mix(moon_ctx *ctx, int dtype, const DecodeMix &p) {
     const int cus = ctx->cu_count > 0 ? ctx->cu_count : 256, per = p.H / p.G, wgs = p.G * mix_head_blocks(per);
     const int n_win = (int)(p.window ? std::min(p.pos + 1, (size_t)p.window) : p.pos + 1), n_keys = n_win + (p.pool ? (int)(p.pos + 1 - n_win) / p.pool : 0);
     if (p.pool && ((p.pos + 1) / p.pool > (size_t)p.blocks || (p.pos + 1 >= (size_t)p.pool && p.pool > p.cap))) return moon_fail(ctx, MOON_EINVAL_DIM, "decode attention: %d pooled blocks kept", p.blocks);
+    if (mix_whole(p) && (p.qk_rms || p.mixes)) return moon_fail(ctx, MOON_EINVAL, "decode attention: norms per head or mixed values beside rotation, blocks or a norm of all of q");
     if (p.dH && (p.dH % p.dG || p.ddimp % 16 || p.dvdimp % 16 || p.ddimp > (int)DELTA_MAX_DIM || p.dvdimp > (int)DELTA_MAX_DIM || p.oc % 8 || p.kd % 64))
         return moon_fail(ctx, MOON_EINVAL_DIM, "decode: delta rule with head sizes %d and %d", p.ddimp, p.dvdimp);
     int S = std::min(std::min((n_keys + MIX_TARGET - 1) / MIX_TARGET, MIX_SPLITS), std::max(1, cus / wgs));

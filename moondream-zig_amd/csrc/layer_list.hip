@@ -477,6 +477,7 @@ static int joined_splits(moon_ctx *ctx, const LayerDev &d, int n, int dp, SegGem
     for (int p = 0; p < n_parts; p++)
         for (int r = 0; r < of[p]; r++) g->kb[s++] = ends[p] + (int)((ends[p + 1] - ends[p]) / 64 * (size_t)r / of[p]) * 64;
     g->kb[s] = d.k0;
+    g->last_first = 1;
     *left = of[0];
     *right = of[1];
     return s;

@@ -113,6 +113,7 @@ struct SegGemm {
     int max_tiles;
     int splits;               // splits > 1: n16 = 0, n32 = N, slab s of c32 (M x ld32 apart) gets k-range s
     int kb[SEG_MAX_SPLITS + 1]; // k-range s is [kb[s], kb[s + 1]), multiples of 64; all zero: even ranges
+    int last_first;           // the last k-range's tiles start first, on every die (where the last ranges are the long ones)
     float softcap;            // > 0: on the f32 segment
 };
 constexpr int SEG_TILE_ROWS = 128; // rows of a tile (both element types walk tile lists of this height)

@@ -19,8 +19,12 @@ __device__ __forceinline__ bool seg_tile(const SegGemm &p, int tile_m, int tile_
     const int tiles_n = (p.N + tile_n - 1) / tile_n;
     const int tiles_m = p.tile_group ? p.max_tiles : (p.M + tile_m - 1) / tile_m;
     const int tiles = tiles_m * tiles_n, total = tiles * p.splits, per_xcd = (total + 7) / 8;
-    const int wg = (blockIdx.x % 8) * per_xcd + blockIdx.x / 8;
-    if ((int)(blockIdx.x / 8) >= per_xcd || wg >= total) return false;
+    int wg = (blockIdx.x % 8) * per_xcd + blockIdx.x / 8;
+    if (p.last_first) { // each XCD: its run of tiles of the last range, then of the one before, ..
+        const int run = (tiles + 7) / 8, j = blockIdx.x / 8, tile = (blockIdx.x % 8) * run + j % run;
+        if (j >= run * p.splits || tile >= tiles) return false;
+        wg = (p.splits - 1 - j / run) * tiles + tile;
+    } else if ((int)(blockIdx.x / 8) >= per_xcd || wg >= total) return false;
     t.split = wg / tiles;
     const int tile = wg % tiles, tn = tile / tiles_m, tm = tile % tiles_m;
     t.n0 = tn * tile_n;
@@ -206,7 +210,7 @@ int launch_seg_gemm(moon_ctx *ctx, int dtype, SegGemm p) {
             return moon_fail(ctx, MOON_EINVAL, "segmented product: %d k splits leave one empty", p.splits);
     const int tile_n = dtype == MOON_DTYPE_BF16 ? BN : 64;
     const size_t tiles = size_t(p.tile_group ? p.max_tiles : (p.M + SEG_TILE_ROWS - 1) / SEG_TILE_ROWS) * ((p.N + tile_n - 1) / tile_n) * p.splits;
-    const dim3 grid((unsigned)((tiles + 7) / 8 * 8));
+    const dim3 grid((unsigned)(p.last_first ? (tiles / p.splits + 7) / 8 * 8 * p.splits : (tiles + 7) / 8 * 8));
     if (dtype == MOON_DTYPE_BF16) {
         const size_t lim = (size_t(1) << 31) - 4096;
         if (size_t(p.a_rows) * p.lda * 2 >= lim || size_t(p.N) * p.K * 2 >= lim)
