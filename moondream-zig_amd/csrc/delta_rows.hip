@@ -25,6 +25,7 @@ constexpr int DC = 16;      // tokens of a chunk
 constexpr int DC_PITCH = DC + 4;
 
 // One chunk and head in the scratch memory, in floats: K' [16][dimp], Q [16][dimp], R^T [dimp][16], G_15 [dimp], P [16][16], V'^T [vdimp][16]
+// (-K' rather than K', so that U is a plain sum)
 __host__ __device__ __forceinline__ size_t chunk_floats(int dimp, int vdimp) { return size_t(49) * dimp + 256 + size_t(16) * vdimp; }
 __host__ __device__ __forceinline__ size_t chunk_lds_floats(int dimp, int vdimp) {
     return size_t(3) * DC * (dimp + 16) + size_t(DC) * vdimp + 2 * DC * DC_PITCH + DC;
@@ -32,7 +33,7 @@ __host__ __device__ __forceinline__ size_t chunk_lds_floats(int dimp, int vdimp)
 
 // Sixteen threads work on a token (and, for A and P, on a token s) until the columns are distributed.
 template <class T>
-__global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaRows p) {
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(6))) void delta_chunk_kernel(DeltaRows p) {
     extern __shared__ __attribute__((aligned(16))) float s_dc[];
     constexpr int PE = Piece<T>::N;
     const int tid = threadIdx.x, lane = tid & 63, tok = tid >> 4, j = tid & 15, chunk = blockIdx.x / p.H, h = blockIdx.x % p.H, c = h / (p.H / p.G);
@@ -164,7 +165,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaRows p) {
             }
             if (is_k) {
 #pragma unroll
-                for (int t = 0; t < DC; t++) o_k[size_t(t) * p.dimp + i] = x[t];
+                for (int t = 0; t < DC; t++) o_k[size_t(t) * p.dimp + i] = -x[t];
             } else store16(o_v + size_t(i - p.dimp) * DC);
         } else { // Q, R and the whole chunk's decay
             const int d = i - p.dimp - p.vdimp;
@@ -192,6 +193,9 @@ constexpr int SCAN_THREADS = 320;
 template <int NT> struct ScanChunk {
     float4_t k[NT], q[NT], r[NT], g[NT], v;
 };
+__device__ __forceinline__ float4_t scan_load(const float *base, unsigned bytes) { // (a base the wavefront shares and 32-bit offsets)
+    return *reinterpret_cast<const float4_t *>(reinterpret_cast<const char *>(base) + bytes);
+}
 template <class T, int NT, int AHEAD>
 __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_scan_kernel(DeltaRows p) {
     __shared__ float4_t s_u[2][4][64], s_o[2][4][64];
@@ -206,13 +210,9 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
     const size_t stride = chunk_floats(p.dimp, p.vdimp);
     const float *src = p.scratch + size_t(h) * chunks * stride;
     if (wave == 4) {
-        const size_t at_p = size_t(49) * p.dimp;
-        float4_t P[AHEAD], V[AHEAD], u_before, p_before;
-        auto request = [&](int a, int chunk) {
-            const float *ap = src + min(chunk, chunks - 1) * stride + at_p;
-            P[a] = *reinterpret_cast<const float4_t *>(ap + col * DC + 4 * quad);
-            V[a] = *reinterpret_cast<const float4_t *>(ap + (DC + v0 + col) * DC + 4 * quad);
-        };
+        float4_t P[AHEAD], u_before, p_before;
+        const unsigned off_p = (49 * p.dimp + col * DC + 4 * quad) * 4;
+        auto request = [&](int a, int chunk) { P[a] = scan_load(src + min(chunk, chunks - 1) * stride, off_p); };
         auto finish = [&](int chunk, int half) { // chunk's parts lie in `half`
             float4_t o = (s_o[half][0][lane] + s_o[half][1][lane]) + (s_o[half][2][lane] + s_o[half][3][lane]);
 #pragma unroll
@@ -228,7 +228,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         auto step = [&](int a, int chunk) {
             const int half = chunk & 1;
             lds_barrier();
-            const float4_t u = V[a] - ((s_u[half][0][lane] + s_u[half][1][lane]) + (s_u[half][2][lane] + s_u[half][3][lane]));
+            const float4_t u = (s_u[half][0][lane] + s_u[half][1][lane]) + (s_u[half][2][lane] + s_u[half][3][lane]);
             if (chunk) finish(chunk - 1, half);
             u_before = u;
             p_before = P[a];
@@ -255,24 +255,32 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
             S[i][e] = p.pos0 && tile < tiles ? state[size_t(16 * tile + 4 * quad + e) * p.vdimp] : 0.0f;
         }
     ScanChunk<NT> ring[AHEAD];
+    unsigned off_k[NT], off_r[NT], off_g[NT];
+#pragma unroll
+    for (int i = 0; i < NT; i++) {
+        const int tile = min(wave + 4 * i, tiles - 1);
+        off_k[i] = (col * p.dimp + 16 * tile + 4 * quad) * 4;
+        off_r[i] = (2 * DC * p.dimp + (16 * tile + col) * DC + 4 * quad) * 4;
+        off_g[i] = (3 * DC * p.dimp + 16 * tile + 4 * quad) * 4;
+    }
+    const unsigned off_v = (49 * p.dimp + (DC + v0 + col) * DC + 4 * quad) * 4;
     auto request = [&](ScanChunk<NT> &b, int chunk) {
         const float *at = src + min(chunk, chunks - 1) * stride;
 #pragma unroll
         for (int i = 0; i < NT; i++) {
-            const int tile = min(wave + 4 * i, tiles - 1);
-            b.k[i] = *reinterpret_cast<const float4_t *>(at + col * p.dimp + 16 * tile + 4 * quad);
-            b.q[i] = *reinterpret_cast<const float4_t *>(at + (DC + col) * p.dimp + 16 * tile + 4 * quad);
-            b.r[i] = *reinterpret_cast<const float4_t *>(at + 2 * DC * p.dimp + (16 * tile + col) * DC + 4 * quad);
-            b.g[i] = *reinterpret_cast<const float4_t *>(at + 3 * DC * p.dimp + 16 * tile + 4 * quad);
+            b.k[i] = scan_load(at, off_k[i]);
+            b.q[i] = scan_load(at + DC * p.dimp, off_k[i]);
+            b.r[i] = scan_load(at, off_r[i]);
+            b.g[i] = scan_load(at, off_g[i]);
         }
-        b.v = *reinterpret_cast<const float4_t *>(at + size_t(49) * p.dimp + (DC + v0 + col) * DC + 4 * quad);
+        b.v = scan_load(at, off_v);
     };
 #pragma unroll
     for (int a = 0; a < AHEAD; a++) request(ring[a], a);
     float4_t o = {0, 0, 0, 0};
     auto step = [&](ScanChunk<NT> &b, int chunk) {
         const int half = chunk & 1;
-        float4_t u = {0, 0, 0, 0};
+        float4_t u = wave == 0 ? b.v : float4_t{0, 0, 0, 0};
 #pragma unroll
         for (int i = 0; i < NT; i++) // (a tile past the end is another wavefront's, with a state of zero here)
 #pragma unroll
@@ -286,7 +294,7 @@ __global__ __launch_bounds__(SCAN_THREADS) __attribute__((amdgpu_waves_per_eu(1,
         for (int i = 0; i < NT; i++)
 #pragma unroll
             for (int j = 0; j < 4; j++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(b.q[i][j], S[i][j], o, 0, 0, 0);
-        u = b.v - ((u0 + u1) + (u2 + u3));
+        u = (u0 + u1) + (u2 + u3);
 #pragma unroll
         for (int i = 0; i < NT; i++) {
             S[i] *= b.g[i];

@@ -206,8 +206,15 @@ __global__ __launch_bounds__(256) void prep_whole_kernel(PrepWhole p) {
         if (i < nq) ss_q += s;
         else if (i < nq + nk) ss_k += s;
     }
-    const float f_q = 1.0f / sqrtf(block_sum(ss_q, sm) / (float)(p.H * p.dim) + p.eps); // (its barriers also order the copy in LDS)
-    const float f_k = p.G ? 1.0f / sqrtf(block_sum(ss_k, sm) / (float)(p.G * p.dim) + p.eps) : 0.0f;
+    ss_q = wave_sum(ss_q);
+    ss_k = wave_sum(ss_k);
+    if ((tid & 63) == 0) {
+        sm[tid >> 6] = ss_q;
+        sm[4 + (tid >> 6)] = ss_k;
+    }
+    lds_barrier(); // (also for the copy in LDS)
+    const float f_q = 1.0f / sqrtf(((sm[0] + sm[1]) + (sm[2] + sm[3])) / (float)(p.H * p.dim) + p.eps);
+    const float f_k = p.G ? 1.0f / sqrtf(((sm[4] + sm[5]) + (sm[6] + sm[7])) / (float)(p.G * p.dim) + p.eps) : 0.0f;
     for (int i = tid * PE; i < nq + nk + nv; i += 256 * PE) {
         const bool is_v = i >= nq + nk, is_q = i < nq;
         const int at = is_q ? i : is_v ? i - nq - nk : i - nq, size = is_v ? p.vdimp : p.dimp, head = at / size, d0 = at % size;
@@ -217,6 +224,36 @@ __global__ __launch_bounds__(256) void prep_whole_kernel(PrepWhole p) {
         const int half = !table ? 0 : (is_v ? p.vdim : p.rot_dims) / 2;
         lm_u32x4 o;
         T *t = reinterpret_cast<T *>(&o);
+        auto weighted = [&](int d, float (&y)[PE]) { // PE elements from d on
+            RowVec<float, 4>::load(x + d, reinterpret_cast<float (&)[4]>(y[0]));
+            if (PE > 4) RowVec<float, 4>::load(x + d + 4, reinterpret_cast<float (&)[4]>(y[PE - 4]));
+#pragma unroll
+            for (int e = 0; e < PE; e++) y[e] *= f;
+            if (!w) return;
+            float a[PE];
+            RowVec<float, 4>::load(w + d, reinterpret_cast<float (&)[4]>(a[0]));
+            if (PE > 4) RowVec<float, 4>::load(w + d + 4, reinterpret_cast<float (&)[4]>(a[PE - 4]));
+#pragma unroll
+            for (int e = 0; e < PE; e++) y[e] *= a[e];
+        };
+        if (d0 >= 2 * half) {
+            float y[PE];
+            weighted(d0, y);
+#pragma unroll
+            for (int e = 0; e < PE; e++) t[e] = (T)y[e];
+        } else if (half % PE == 0) { // the other halves of the pairs lie side by side, too
+            const bool first = d0 < half;
+            float y[PE], z[PE];
+            weighted(d0, y);
+            weighted(first ? d0 + half : d0 - half, z);
+            const float4_t *cs = reinterpret_cast<const float4_t *>(table + size_t(pos) * half + (first ? d0 : d0 - half)); // two pairs each
+#pragma unroll
+            for (int e = 0; e < PE; e += 2) {
+                const float4_t c = cs[e / 2];
+                t[e] = (T)(first ? y[e] * c[0] - z[e] * c[1] : y[e] * c[0] + z[e] * c[1]);
+                t[e + 1] = (T)(first ? y[e + 1] * c[2] - z[e + 1] * c[3] : y[e + 1] * c[2] + z[e + 1] * c[3]);
+            }
+        } else
 #pragma unroll
         for (int e = 0; e < PE; e++) {
             const int d = d0 + e;
